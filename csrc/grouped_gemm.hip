@@ -94,6 +94,8 @@ __device__ __forceinline__ const bf16x8* gg_frag(const u16* lds, int row,
 // MODE=2: rows gathered, one B stream, relu(x)^2 in the epilogue.
 // MODE=3: like MODE=1 with the clamped unit g sigmoid(1.702 g) (u + 1),
 // g = min(gate, limit), u = clamp(up, -limit, limit).
+// MODE=4: like MODE=1 with both products of row r times row_w[r] first (the
+// expert reads row_w * x).
 // Waves arranged WROWS(M) x WCOLS(N); wave tile = (BM/WROWS) x (BN/WCOLS).
 template <int MODE, int BM, int BN, int WROWS, int WCOLS>
 __global__ __launch_bounds__(WROWS* WCOLS * 64) void grouped_gemm_kernel(
@@ -103,8 +105,9 @@ __global__ __launch_bounds__(WROWS* WCOLS * 64) void grouped_gemm_kernel(
     const int* __restrict__ row_tok,    // [rows_max] or nullptr
     const int* __restrict__ tile_off,   // [E+1] padded-offset / BM
     const int* __restrict__ counts,     // [E] live rows per expert
-    int n_experts, int n_cols, long K, float limit) {
-  constexpr bool GATED = MODE == 1 || MODE == 3;  // two B streams (gate, up)
+    int n_experts, int n_cols, long K, float limit,
+    const float* __restrict__ row_w) {  // [rows_max], MODE 4
+  constexpr bool GATED = MODE == 1 || MODE >= 3;  // two B streams (gate, up)
   constexpr bool GATHER = MODE != 0;  // A rows come through row_tok
   constexpr int WAVES = WROWS * WCOLS;
   constexpr int WM = BM / WROWS;
@@ -224,6 +227,11 @@ __global__ __launch_bounds__(WROWS* WCOLS * 64) void grouped_gemm_kernel(
           const float g = v;
           v = g / (1.0f + __expf(-g)) * accu[i][j][r];
         }
+        if (MODE == 4) {
+          const float rw = row_w[seg0 + m0 + grow];
+          const float g = v * rw;
+          v = g / (1.0f + __expf(-g)) * (accu[i][j][r] * rw);
+        }
         if (MODE == 3) {
           const float g = fminf(v, limit);
           const float u = fminf(fmaxf(accu[i][j][r], -limit), limit);
@@ -244,7 +252,7 @@ static void grouped_gemm_launch(void* out, const void* a, const void* w,
                                 const int* counts, int n_experts,
                                 int max_tiles, int n_cols, long K,
                                 int gate_silu, int bm, float limit,
-                                hipStream_t stream) {
+                                const float* row_w, hipStream_t stream) {
   if (max_tiles == 0) return;
 #define GG_LAUNCH(GS, BM, BN, WR, WC)                                       \
   {                                                                         \
@@ -253,7 +261,7 @@ static void grouped_gemm_launch(void* out, const void* a, const void* w,
     hipLaunchKernelGGL((grouped_gemm_kernel<GS, BM, BN, WR, WC>), grid,     \
                        block, 0, stream, (u16*)out, (const u16*)a,          \
                        (const u16*)w, row_tok, tile_off, counts, n_experts, \
-                       n_cols, K, limit);                                   \
+                       n_cols, K, limit, row_w);                            \
     return;                                                                 \
   }
   /* no hipGetLastError in this launcher: error-state queries are rejected
@@ -261,17 +269,20 @@ static void grouped_gemm_launch(void* out, const void* a, const void* w,
   if (bm == 128 && n_cols % 128 == 0) {
     if (gate_silu == 1) GG_LAUNCH(1, 128, 128, 2, 4)
     else if (gate_silu == 3) GG_LAUNCH(3, 128, 128, 2, 4)
+    else if (gate_silu == 4) GG_LAUNCH(4, 128, 128, 2, 4)
     else if (gate_silu == 2) GG_LAUNCH(2, 128, 128, 2, 4)
     else GG_LAUNCH(0, 128, 128, 2, 4)
   }
   if (bm == 128) {
     if (gate_silu == 1) GG_LAUNCH(1, 128, 64, 4, 2)
     else if (gate_silu == 3) GG_LAUNCH(3, 128, 64, 4, 2)
+    else if (gate_silu == 4) GG_LAUNCH(4, 128, 64, 4, 2)
     else if (gate_silu == 2) GG_LAUNCH(2, 128, 64, 4, 2)
     else GG_LAUNCH(0, 128, 64, 4, 2)
   }
   if (gate_silu == 1) GG_LAUNCH(1, 64, 64, 2, 2)
   else if (gate_silu == 3) GG_LAUNCH(3, 64, 64, 2, 2)
+  else if (gate_silu == 4) GG_LAUNCH(4, 64, 64, 2, 2)
   else if (gate_silu == 2) GG_LAUNCH(2, 64, 64, 2, 2)
   else GG_LAUNCH(0, 64, 64, 2, 2)
 #undef GG_LAUNCH
@@ -284,7 +295,8 @@ extern "C" void sutro_grouped_gemm(void* out, const void* a, const void* w,
                                    int gate_silu, int bm,
                                    hipStream_t stream) {
   grouped_gemm_launch(out, a, w, row_tok, tile_off, counts, n_experts,
-                      max_tiles, n_cols, K, gate_silu, bm, 0.f, stream);
+                      max_tiles, n_cols, K, gate_silu, bm, 0.f, nullptr,
+                      stream);
 }
 
 // the clamped gated unit (mode 3) with its limit
@@ -295,7 +307,16 @@ extern "C" void sutro_grouped_gemm_glu(void* out, const void* a, const void* w,
                                        int bm, float limit,
                                        hipStream_t stream) {
   grouped_gemm_launch(out, a, w, row_tok, tile_off, counts, n_experts,
-                      max_tiles, n_cols, K, 3, bm, limit, stream);
+                      max_tiles, n_cols, K, 3, bm, limit, nullptr, stream);
+}
+
+// the silu unit over weighted rows (mode 4)
+extern "C" void sutro_grouped_gemm_weighted(
+    void* out, const void* a, const void* w, const int* row_tok,
+    const int* tile_off, const int* counts, int n_experts, int max_tiles,
+    int n_cols, long K, int bm, const float* row_w, hipStream_t stream) {
+  grouped_gemm_launch(out, a, w, row_tok, tile_off, counts, n_experts,
+                      max_tiles, n_cols, K, 4, bm, 0.f, row_w, stream);
 }
 
 // ---- fused MoE combine: out[t] = sum_j w[t,j] * rows[padpos[t,j]] ----

@@ -8,7 +8,10 @@
 //   local_attention  softmax attention of every new token over the cached
 //                    keys its mask lets it see, times a per-head sigmoid gate;
 //                    optionally r1[h] * ln(1 + r2[h] * distance) is taken off
-//                    every score (per-head logarithmic distance bias).
+//                    every score (per-head logarithmic distance bias); the
+//                    gate may be one number per head or one per element, and
+//                    a sink (a score without key or value: 0, or a number per
+//                    head) may join the softmax denominator.
 //
 // Cache layout per layer: K [blocks, G, page, dk], V [blocks, G, page, ldv]
 // of which the first dv columns of a row are the value (a shared latent is key
@@ -238,9 +241,10 @@ __global__ void local_attention_kernel(
     const int* __restrict__ bt, int bt_stride, const int* __restrict__ seq_lens,
     const int* __restrict__ qlocs, const int* __restrict__ token_seq,
     float scale, int chunk, int window, const A* __restrict__ proj, long ld,
-    int gate_off, float out_scale, const float* __restrict__ bias_r1,
-    const float* __restrict__ bias_r2, int sink, int keep_first, long t0, long T, int H, int G,
-    int dk, int dv, int ldv, int page) {
+    int gate_off, int gate_n, float out_scale,
+    const float* __restrict__ bias_r1, const float* __restrict__ bias_r2,
+    int sink, const float* __restrict__ sink_w, int keep_first, long t0,
+    long T, int H, int G, int dk, int dv, int ldv, int page) {
   extern __shared__ float sm[];  // WPB * dk floats: the wave's query
   const int lane = threadIdx.x & (WAVE - 1);
   const int wid = threadIdx.x / WAVE;
@@ -270,8 +274,8 @@ __global__ void local_attention_kernel(
   const float r1 = bias_r1 ? bias_r1[h] : 0.f;
   const float r2 = bias_r1 ? bias_r2[h] : 0.f;
 
-  // a sink is a key of score 0 without a value that is always visible
-  float m = sink ? 0.f : -INFINITY, l = sink ? 1.f : 0.f;
+  // a sink is a score without a key or value that is always visible
+  float m = sink ? (sink_w ? sink_w[h] : 0.f) : -INFINITY, l = sink ? 1.f : 0.f;
   float acc[NV];
 #pragma unroll
   for (int c = 0; c < NV; ++c) acc[c] = 0.f;
@@ -311,14 +315,17 @@ __global__ void local_attention_kernel(
       }
     }
   }
-  float gate = out_scale;
-  if (gate_off >= 0) gate *= sigmoid_f(ldf<A>(proj + t * ld + gate_off + h));
-  const float f = gate / l;
+  const A* gp = gate_off >= 0 ? proj + t * ld + gate_off + (long)h * gate_n
+                              : nullptr;
+  float f = out_scale / l;
+  if (gp && gate_n == 1) f *= sigmoid_f(ldf<A>(gp));
 #pragma unroll
   for (int c = 0; c < NV; ++c) {
     const int col = lane + c * (int)WAVE;
-    if (col < dv)
-      stf<A>(out + t * ldo + out_off + (long)h * dv + col, acc[c] * f);
+    if (col >= dv) continue;
+    float o = acc[c] * f;
+    if (gp && gate_n > 1) o *= sigmoid_f(ldf<A>(gp + col));
+    stf<A>(out + t * ldo + out_off + (long)h * dv + col, o);
   }
 }
 
@@ -349,9 +356,10 @@ __global__ void __launch_bounds__(NW * 64) local_attention_rows_kernel(
     const int* __restrict__ bt, int bt_stride, const int* __restrict__ seq_lens,
     const int* __restrict__ qlocs, const int* __restrict__ token_seq,
     float scale, int chunk, int window, const A* __restrict__ proj, long ld,
-    int gate_off, float out_scale, const float* __restrict__ bias_r1,
-    const float* __restrict__ bias_r2, int sink, int keep_first, long t0, int H, int G, int dk,
-    int dv, int ldv, int page) {
+    int gate_off, int gate_n, float out_scale,
+    const float* __restrict__ bias_r1, const float* __restrict__ bias_r2,
+    int sink, const float* __restrict__ sink_w, int keep_first, long t0, int H,
+    int G, int dk, int dv, int ldv, int page) {
   typedef typename Vec16<A>::type vec_t;
   constexpr int EPL = 16 / sizeof(A);     // elements per lane
   constexpr int KPI = 64 / LPR;           // keys per load instruction
@@ -475,21 +483,24 @@ __global__ void __launch_bounds__(NW * 64) local_attention_rows_kernel(
   float mx = comb[0];  // wave 0 always has a tile
 #pragma unroll
   for (int w = 1; w < NW; ++w) mx = fmaxf(mx, comb[w * CS]);
-  // a sink (score 0, no value) joins the normalisation here, once per row
-  if (sink) mx = fmaxf(mx, 0.f);
-  float wgt[NW], lsum = sink ? expf(-mx) : 0.f;
+  // a sink (a score, no value) joins the normalisation here, once per row
+  const float sk = sink && sink_w ? sink_w[h] : 0.f;
+  if (sink) mx = fmaxf(mx, sk);
+  float wgt[NW], lsum = sink ? expf(sk - mx) : 0.f;
 #pragma unroll
   for (int w = 0; w < NW; ++w) {
     wgt[w] = expf(comb[w * CS] - mx);   // a wave without tiles: exp(-inf) = 0
     lsum += wgt[w] * comb[w * CS + 1];
   }
-  float gate = out_scale;
-  if (gate_off >= 0) gate *= sigmoid_f(ldf<A>(proj + t * ld + gate_off + h));
-  const float f = gate / lsum;
+  const A* gp = gate_off >= 0 ? proj + t * ld + gate_off + (long)h * gate_n
+                              : nullptr;
+  float f = out_scale / lsum;
+  if (gp && gate_n == 1) f *= sigmoid_f(ldf<A>(gp));
   for (int c = threadIdx.x; c < dv; c += blockDim.x) {
     float o = 0.f;
 #pragma unroll
     for (int w = 0; w < NW; ++w) o += wgt[w] * comb[w * CS + 2 + c];
+    if (gp && gate_n > 1) f = out_scale / lsum * sigmoid_f(ldf<A>(gp + c));
     stf<A>(out + t * ldo + out_off + (long)h * dv + c, o * f);
   }
 }
@@ -549,10 +560,10 @@ static void launch_local_attention(
     void* out, long ldo, int out_off, const void* q, const void* k_cache,
     const void* v_cache, const int* bt, int bt_stride, const int* seq_lens,
     const int* qlocs, const int* token_seq, float scale, int chunk,
-    int window, const void* proj, long ld, int gate_off, float out_scale,
-    const float* bias_r1, const float* bias_r2, int sink, int keep_first,
-    long t0, long T,
-    int H, int G, int dk, int dv, int ldv, int page, hipStream_t s) {
+    int window, const void* proj, long ld, int gate_off, int gate_n,
+    float out_scale, const float* bias_r1, const float* bias_r2, int sink,
+    const float* sink_w, int keep_first, long t0, long T, int H, int G, int dk,
+    int dv, int ldv, int page, hipStream_t s) {
   const long units = T * H;
   const int grid = (int)((units + WPB - 1) / WPB);
   if (grid == 0) return;
@@ -575,8 +586,8 @@ static void launch_local_attention(
                      ldo, out_off, (const A*)q, (const A*)k_cache,            \
                      (const A*)v_cache, bt, bt_stride, seq_lens, qlocs,       \
                      token_seq, scale, chunk, window, (const A*)proj, ld,     \
-                     gate_off, out_scale, bias_r1, bias_r2, sink, keep_first, t0, H, G,   \
-                     dk, dv, ldv, page)
+                     gate_off, gate_n, out_scale, bias_r1, bias_r2, sink,     \
+                     sink_w, keep_first, t0, H, G, dk, dv, ldv, page)
       if (lpr == 2) LAUNCH_LR(2);
       else if (lpr == 4) LAUNCH_LR(4);
       else if (lpr == 8) LAUNCH_LR(8);
@@ -594,8 +605,9 @@ static void launch_local_attention(
                      dim3(WPB * WAVE), smem, s, (A*)out, ldo, out_off,       \
                      (const A*)q, (const A*)k_cache, (const A*)v_cache, bt,  \
                      bt_stride, seq_lens, qlocs, token_seq, scale, chunk,    \
-                     window, (const A*)proj, ld, gate_off, out_scale,        \
-                     bias_r1, bias_r2, sink, keep_first, t0, T, H, G, dk, dv, ldv, page)
+                     window, (const A*)proj, ld, gate_off, gate_n, out_scale,\
+                     bias_r1, bias_r2, sink, sink_w, keep_first, t0, T, H, G,\
+                     dk, dv, ldv, page)
   if (dv <= 64) LAUNCH_LA(1);
   else if (dv <= 128) LAUNCH_LA(2);
   else if (dv <= 256) LAUNCH_LA(4);
@@ -607,20 +619,21 @@ extern "C" void mix_local_attention(
     void* out, long ldo, int out_off, const void* q, const void* k_cache,
     const void* v_cache, const int* bt, int bt_stride, const int* seq_lens,
     const int* qlocs, const int* token_seq, float scale, int chunk,
-    int window, const void* proj, long ld, int gate_off, float out_scale,
-    const float* bias_r1, const float* bias_r2, int sink, int keep_first,
-    long t0, long T,
-    int H, int G, int dk, int dv, int ldv, int page, int f32, hipStream_t s) {
+    int window, const void* proj, long ld, int gate_off, int gate_n,
+    float out_scale, const float* bias_r1, const float* bias_r2, int sink,
+    const float* sink_w, int keep_first, long t0, long T, int H, int G, int dk,
+    int dv, int ldv, int page, int f32, hipStream_t s) {
   if (f32)
     launch_local_attention<float>(out, ldo, out_off, q, k_cache, v_cache, bt,
                                   bt_stride, seq_lens, qlocs, token_seq, scale,
-                                  chunk, window, proj, ld, gate_off, out_scale,
-                                  bias_r1, bias_r2, sink, keep_first, t0, T, H, G, dk, dv,
-                                  ldv, page, s);
+                                  chunk, window, proj, ld, gate_off, gate_n,
+                                  out_scale, bias_r1, bias_r2, sink, sink_w,
+                                  keep_first, t0, T, H, G, dk, dv, ldv, page,
+                                  s);
   else
     launch_local_attention<u16>(out, ldo, out_off, q, k_cache, v_cache, bt,
                                 bt_stride, seq_lens, qlocs, token_seq, scale,
-                                chunk, window, proj, ld, gate_off, out_scale,
-                                bias_r1, bias_r2, sink, keep_first, t0, T, H, G, dk, dv,
-                                ldv, page, s);
+                                chunk, window, proj, ld, gate_off, gate_n,
+                                out_scale, bias_r1, bias_r2, sink, sink_w,
+                                keep_first, t0, T, H, G, dk, dv, ldv, page, s);
 }

@@ -11,9 +11,11 @@
 //     tile's first row are never read; masked scores contribute exactly 0,
 //   - an optional per-head distance bias r1 * ln(1 + r2 * (p - j)) taken off
 //     the scaled score,
-//   - score scale from the caller, per-head sigmoid output gate and output
-//     scale in the epilogue, output written into a column section of the
-//     merged output-projection input.
+//   - an optional sink (a score without key or value, 0 or one a head) in the
+//     softmax denominator,
+//   - score scale from the caller, sigmoid output gate (one a head or one an
+//     element) and output scale in the epilogue, output written into a column
+//     section of the merged output-projection input.
 //
 // Fragment layouts (gfx950 v_mfma_f32_32x32x16_bf16):
 //   A[32,16]: lane l holds A[l%32][(l/32)*8 + j], j = 0..7
@@ -51,9 +53,11 @@ local_attention_mfma_kernel(
     const int* __restrict__ bt, int bt_stride, const int* __restrict__ seq_lens,
     const int* __restrict__ qlocs, const int* __restrict__ tile_seq,
     const int* __restrict__ tile_q0, float scale, int chunk, int window,
-    const u16* __restrict__ proj, long ld, int gate_off, float out_scale,
-    const float* __restrict__ bias_r1, const float* __restrict__ bias_r2,
-    int sink, int keep_first, int H, int Hk, int dk, int dv, int ldv, int parts) {
+    const u16* __restrict__ proj, long ld, int gate_off, int gate_n,
+    float out_scale, const float* __restrict__ bias_r1,
+    const float* __restrict__ bias_r2, int sink,
+    const float* __restrict__ sink_w, int keep_first, int H, int Hk, int dk,
+    int dv, int ldv, int parts) {
   const int lane = threadIdx.x & (WAVE - 1);
   const int w = threadIdx.x / WAVE;
   const int G = blockDim.x / WAVE;        // query heads of this workgroup
@@ -102,9 +106,10 @@ local_attention_mfma_kernel(
   f32x16 acc[DVP / 32];
 #pragma unroll
   for (int b = 0; b < DVP / 32; ++b) acc[b] = (f32x16)(0.f);
-  // a sink (a key of score 0 without a value) starts the running maximum at
-  // 0 and the running sum at its weight
-  float m_run = sink ? 0.f : -1e30f, l_run = sink ? 1.f : 0.f;
+  // a sink (a score without key or value) starts the running maximum at its
+  // score and the running sum at its weight
+  float m_run = sink ? (sink_w ? sink_w[hq] : 0.f) : -1e30f;
+  float l_run = sink ? 1.f : 0.f;
   // distance bias of this wave's head: r1 * ln(1 + r2 * (p - j))
   const float r1 = bias_r1 ? bias_r1[hq] : 0.f;
   const float r2 = bias_r1 ? bias_r2[hq] : 0.f;
@@ -204,7 +209,7 @@ local_attention_mfma_kernel(
   // epilogue: out = acc / l * out_scale * sigmoid(gate logit of (row, head))
   if (hi == 0) {
     float f = l_run > 0.f ? out_scale / l_run : 0.f;
-    if (gate_off >= 0 && my_q < nq)
+    if (gate_off >= 0 && gate_n == 1 && my_q < nq)
       f *= sigmoid_f(bf2f(proj[(long)(row_base + my_q) * ld + gate_off + hq]));
     fin_lds[my_q] = f;
   }
@@ -219,9 +224,14 @@ local_attention_mfma_kernel(
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
         const int qrow = drow(r, hi);
-        if (qrow < nq)
+        if (qrow < nq) {
+          float o = acc[b][r] * fin[r];
+          if (gate_off >= 0 && gate_n > 1)
+            o *= sigmoid_f(bf2f(proj[(long)(row_base + qrow) * ld + gate_off +
+                                     (long)hq * gate_n + col]));
           out[(long)(row_base + qrow) * ldo + out_off + (long)hq * dv + col] =
-              f2bf(acc[b][r] * fin[r]);
+              f2bf(o);
+        }
       }
     }
   }
@@ -233,9 +243,9 @@ extern "C" int mix_local_attention_mfma(
     const void* v_cache, const int* bt, int bt_stride, const int* seq_lens,
     const int* qlocs, const int* tile_seq, const int* tile_q0, int n_tiles,
     float scale, int chunk, int window, const void* proj, long ld,
-    int gate_off, float out_scale, const float* bias_r1, const float* bias_r2,
-    int sink, int keep_first, int H, int Hk, int dk, int dv, int ldv, int page,
-    hipStream_t s) {
+    int gate_off, int gate_n, float out_scale, const float* bias_r1,
+    const float* bias_r2, int sink, const float* sink_w, int keep_first, int H,
+    int Hk, int dk, int dv, int ldv, int page, hipStream_t s) {
   if (page != PG || dk % 8 || dv % 8 || ldv % 8 || dk > 256 || dv > 256 || H % Hk)
     return 0;
   const int DKP = dk <= 64 ? 64 : (dk <= 128 ? 128 : 256);
@@ -260,8 +270,9 @@ extern "C" int mix_local_attention_mfma(
                      ldo, out_off, (const u16*)q, (const u16*)k_cache,        \
                      (const u16*)v_cache, bt, bt_stride, seq_lens, qlocs,     \
                      tile_seq, tile_q0, scale, chunk, window,                 \
-                     (const u16*)proj, ld, gate_off, out_scale, bias_r1,     \
-                     bias_r2, sink, keep_first, H, Hk, dk, dv, ldv, parts)
+                     (const u16*)proj, ld, gate_off, gate_n, out_scale,       \
+                     bias_r1, bias_r2, sink, sink_w, keep_first, H, Hk, dk,   \
+                     dv, ldv, parts)
   if (DKP == 64) {
     if (DVP == 64) LAUNCH_M(64, 64);
     else if (DVP == 128) LAUNCH_M(64, 128);

@@ -50,14 +50,15 @@ void mix_attn_prep(void*, const void*, long, int, int, int, const float*,
 void mix_local_attention(void*, long, int, const void*, const void*,
                          const void*, const int*, int, const int*, const int*,
                          const int*, float, int, int, const void*, long, int,
-                         float, const float*, const float*, int, int, long,
-                         long, int, int, int, int, int, int, int, hipStream_t);
+                         int, float, const float*, const float*, int,
+                         const float*, int, long, long, int, int, int, int,
+                         int, int, int, hipStream_t);
 int mix_local_attention_mfma(void*, long, int, const void*, const void*,
                              const void*, const int*, int, const int*,
                              const int*, const int*, const int*, int, float,
-                             int, int, const void*, long, int, float,
-                             const float*, const float*, int, int, int, int,
-                             int, int, int, int, hipStream_t);
+                             int, int, const void*, long, int, int, float,
+                             const float*, const float*, int, const float*,
+                             int, int, int, int, int, int, int, hipStream_t);
 int mix_latent_splits(long, int, int, int, int, int, int);
 int mix_latent_attention(void*, long, int, const void*, const void*,
                          const int*, int, const int*, const int*, const int*,
@@ -72,13 +73,23 @@ void mix_dyt_residual(float*, const void*, const float*, const void*,
                       const float*, const float*, const float*, void*, long,
                       int, int, hipStream_t);
 void mix_moe_route(int*, float*, const float*, long, int, int, int, int, int,
-                   hipStream_t);
+                   int, hipStream_t);
 void mix_moe_dispatch(int*, int*, int*, int*, const int*, const long*, long,
-                      int, int, int, long, int*, hipStream_t);
+                      int, int, int, long, int*, const float*, float*,
+                      hipStream_t);
 long mix_moe_dispatch_scratch(long, int);
 void mix_expert_gemm_plain(void*, const void*, const void*, const int*,
                            const int*, const int*, int, int, int, int, long,
-                           int, float, int, hipStream_t);
+                           int, float, const float*, int, hipStream_t);
+void sutro_grouped_gemm_weighted(void*, const void*, const void*, const int*,
+                                 const int*, const int*, int, int, int, long,
+                                 int, const float*, hipStream_t);
+long mix_hyper_lds(int, int);
+int mix_hyper_rmsnorm(float*, const float*, const void*, const void*,
+                      const int*, const float*, float, int, const void*,
+                      const float*, const float*, const float*, const float*,
+                      float, void*, int, long, int, int, int, hipStream_t);
+void mix_relu_sq(void*, long, int, hipStream_t);
 void sutro_grouped_gemm_glu(void*, const void*, const void*, const int*,
                             const int*, const int*, int, int, int, long, int,
                             float, hipStream_t);
@@ -100,8 +111,8 @@ void mix_rotary_sections(float*, const void*, long, int, int, int,
                          const float*, int, float, long, int, int, int, int,
                          hipStream_t);
 void mix_latent_prep(void*, const long*, const void*, long, int, const float*,
-                     float, const float*, int, int, const void*, long, long,
-                     void*, long, int, int, hipStream_t);
+                     float, const float*, int, int, int, const void*, long,
+                     long, void*, long, int, int, hipStream_t);
 void mix_rope_table(float*, const long*, const float*, int, float, long,
                     hipStream_t);
 void mix_ssd_prep(float*, float*, float*, const void*, long, int, int,
@@ -269,7 +280,8 @@ void local_attention(torch::Tensor out, long out_off, torch::Tensor q,
                      c10::optional<torch::Tensor> tile_q0,
                      long prefill_rows, c10::optional<torch::Tensor> bias_r1,
                      c10::optional<torch::Tensor> bias_r2, bool sink,
-                     long keep_first) {
+                     long keep_first, long gate_n,
+                     c10::optional<torch::Tensor> sink_w) {
   CHECK_GPU(q); CHECK_CONTIG(q); CHECK_CONTIG(k_cache); CHECK_GPU(v_cache);
   CHECK_I32(bt); CHECK_I32(seq_lens); CHECK_I32(qlocs); CHECK_I32(token_seq);
   CHECK_CONTIG(bt);
@@ -302,8 +314,15 @@ void local_attention(torch::Tensor out, long out_off, torch::Tensor q,
               proj.scalar_type() == q.scalar_type(), "dtype mismatch");
   TORCH_CHECK(token_seq.numel() == T && qlocs.numel() == seq_lens.numel() + 1 &&
               bt.size(0) == seq_lens.numel(), "batch metadata sizes");
-  if (gate_off >= 0) check_proj(proj, gate_off, H, "gate");
+  TORCH_CHECK(gate_n == 1 || gate_n == dv, "one gate a head or an element");
+  if (gate_off >= 0) check_proj(proj, gate_off, H * gate_n, "gate");
   TORCH_CHECK(proj.size(0) == T, "row mismatch");
+  const float* sw = nullptr;
+  if (sink_w.has_value()) {
+    CHECK_GPU(*sink_w); CHECK_F32(*sink_w); CHECK_CONTIG(*sink_w);
+    TORCH_CHECK(sink && sink_w->numel() == H, "sink: one score per head");
+    sw = sink_w->data_ptr<float>();
+  }
   // one shared latent per token (the value is the head of the key row): rows
   // of all heads share the matrix-core tiles, single tokens included
   const bool shared_latent =
@@ -360,9 +379,9 @@ void local_attention(torch::Tensor out, long out_off, torch::Tensor q,
             (int)bt.size(1), seq_lens.data_ptr<int>(), qlocs.data_ptr<int>(),
             tile_seq->data_ptr<int>(), tile_q0->data_ptr<int>(),
             (int)tile_seq->numel(), (float)scale, (int)chunk, (int)window,
-            proj.data_ptr(), proj.stride(0), (int)gate_off, (float)out_scale,
-            r1, r2, sink ? 1 : 0, (int)keep_first, (int)H, (int)G, (int)dk,
-            (int)dv, (int)ldv, (int)page, cur_stream()))
+            proj.data_ptr(), proj.stride(0), (int)gate_off, (int)gate_n,
+            (float)out_scale, r1, r2, sink ? 1 : 0, sw, (int)keep_first, (int)H,
+            (int)G, (int)dk, (int)dv, (int)ldv, (int)page, cur_stream()))
       t0 = prefill_rows;
   }
   if (t0 < T)
@@ -372,8 +391,8 @@ void local_attention(torch::Tensor out, long out_off, torch::Tensor q,
                         seq_lens.data_ptr<int>(), qlocs.data_ptr<int>(),
                         token_seq.data_ptr<int>(), (float)scale, (int)chunk,
                         (int)window, proj.data_ptr(), proj.stride(0),
-                        (int)gate_off, (float)out_scale, r1, r2, sink ? 1 : 0,
-                        (int)keep_first, t0, T - t0, (int)H,
+                        (int)gate_off, (int)gate_n, (float)out_scale, r1, r2,
+                        sink ? 1 : 0, sw, (int)keep_first, t0, T - t0, (int)H,
                         (int)G, (int)dk, (int)dv, (int)ldv, (int)page,
                         act_kind(q), cur_stream());
 }
@@ -807,7 +826,7 @@ void dyt_residual(torch::Tensor x, c10::optional<torch::Tensor> y1,
 }
 
 void moe_route(torch::Tensor idx, torch::Tensor wts, torch::Tensor logits,
-               long groups, long keep, long rank) {
+               long groups, long keep, long rank, bool renorm) {
   CHECK_GPU(logits); CHECK_F32(logits); CHECK_CONTIG(logits);
   CHECK_GPU(idx); CHECK_I32(idx); CHECK_CONTIG(idx);
   CHECK_GPU(wts); CHECK_F32(wts); CHECK_CONTIG(wts);
@@ -821,12 +840,14 @@ void moe_route(torch::Tensor idx, torch::Tensor wts, torch::Tensor logits,
   TORCH_CHECK(4 * (E + groups) * 4 <= 64 * 1024, "too many experts");
   mix_moe_route(idx.data_ptr<int>(), wts.data_ptr<float>(),
                 logits.data_ptr<float>(), T, (int)E, (int)top, (int)groups,
-                (int)keep, (int)rank, cur_stream());
+                (int)keep, (int)rank, renorm ? 1 : 0, cur_stream());
 }
 
 void moe_dispatch(torch::Tensor row_tok, torch::Tensor tile_off,
                   torch::Tensor counts, torch::Tensor padpos,
-                  torch::Tensor idx, long bm) {
+                  torch::Tensor idx, long bm,
+                  c10::optional<torch::Tensor> wts,
+                  c10::optional<torch::Tensor> row_w) {
   CHECK_GPU(idx); CHECK_I32(idx); CHECK_CONTIG(idx);
   CHECK_GPU(row_tok); CHECK_I32(row_tok); CHECK_CONTIG(row_tok);
   CHECK_GPU(tile_off); CHECK_I32(tile_off); CHECK_CONTIG(tile_off);
@@ -839,6 +860,13 @@ void moe_dispatch(torch::Tensor row_tok, torch::Tensor tile_off,
               row_tok.numel() >= T * k + E * (bm - 1), "segment table sizes");
   TORCH_CHECK((2 * E + 1) * 4 <= 64 * 1024 && T * k < (1L << 31),
               "too many experts or pairs");
+  if (row_w.has_value()) {
+    TORCH_CHECK(wts.has_value(), "row weights come from pair weights");
+    CHECK_GPU(*wts); CHECK_F32(*wts); CHECK_CONTIG(*wts);
+    CHECK_GPU(*row_w); CHECK_F32(*row_w); CHECK_CONTIG(*row_w);
+    TORCH_CHECK(wts->sizes() == idx.sizes() &&
+                row_w->numel() == row_tok.numel(), "weight shapes");
+  }
   torch::Tensor buf;
   int* scratch = nullptr;
   if (const long n = mix_moe_dispatch_scratch(T * k, (int)E)) {
@@ -848,7 +876,10 @@ void moe_dispatch(torch::Tensor row_tok, torch::Tensor tile_off,
   mix_moe_dispatch(row_tok.data_ptr<int>(), tile_off.data_ptr<int>(),
                    counts.data_ptr<int>(), padpos.data_ptr<int>(),
                    idx.data_ptr<int>(), nullptr, T * k, (int)k, (int)E,
-                   (int)bm, row_tok.numel(), scratch, cur_stream());
+                   (int)bm, row_tok.numel(), scratch,
+                   row_w.has_value() ? wts->data_ptr<float>() : nullptr,
+                   row_w.has_value() ? row_w->data_ptr<float>() : nullptr,
+                   cur_stream());
 }
 
 // choices of token t: row ids[t] of `table` [vocab, k] (entries checked when
@@ -880,12 +911,14 @@ void moe_dispatch_table(torch::Tensor row_tok, torch::Tensor tile_off,
   mix_moe_dispatch(row_tok.data_ptr<int>(), tile_off.data_ptr<int>(),
                    counts.data_ptr<int>(), padpos.data_ptr<int>(),
                    table.data_ptr<int>(), ids.data_ptr<long>(), T * k, (int)k,
-                   (int)E, (int)bm, row_tok.numel(), scratch, cur_stream());
+                   (int)E, (int)bm, row_tok.numel(), scratch, nullptr, nullptr,
+                   cur_stream());
 }
 
 void expert_gemm(torch::Tensor out, torch::Tensor a, torch::Tensor w,
                  c10::optional<torch::Tensor> row_tok, torch::Tensor tile_off,
-                 torch::Tensor counts, long act, long bm, double limit) {
+                 torch::Tensor counts, long act, long bm, double limit,
+                 c10::optional<torch::Tensor> row_w) {
   CHECK_GPU(a); CHECK_CONTIG(a); CHECK_GPU(w); CHECK_CONTIG(w);
   CHECK_GPU(out); CHECK_CONTIG(out);
   CHECK_I32(tile_off); CHECK_I32(counts); CHECK_GPU(tile_off); CHECK_GPU(counts);
@@ -916,8 +949,21 @@ void expert_gemm(torch::Tensor out, torch::Tensor a, torch::Tensor w,
   }
   TORCH_CHECK((act != 0) == (rt != nullptr),
               "the gathered stage carries the activation");
-  if (kind == 0 && K % 64 == 0 && N % 64 == 0) {
-    if (act == 3)
+  const float* rw = nullptr;
+  if (row_w.has_value()) {
+    CHECK_GPU(*row_w); CHECK_F32(*row_w); CHECK_CONTIG(*row_w);
+    TORCH_CHECK(act != 0 && row_w->numel() == n_rows,
+                "row weights go with the gathered stage");
+    rw = row_w->data_ptr<float>();
+  }
+  // weighted rows: the matrix-core kernel has the silu unit only
+  if (kind == 0 && K % 64 == 0 && N % 64 == 0 && (!rw || act == 1)) {
+    if (rw)
+      sutro_grouped_gemm_weighted(
+          out.data_ptr(), a.data_ptr(), w.data_ptr(), rt,
+          tile_off.data_ptr<int>(), counts.data_ptr<int>(), (int)E,
+          (int)(n_rows / bm), (int)N, K, (int)bm, rw, cur_stream());
+    else if (act == 3)
       sutro_grouped_gemm_glu(out.data_ptr(), a.data_ptr(), w.data_ptr(), rt,
                              tile_off.data_ptr<int>(), counts.data_ptr<int>(),
                              (int)E, (int)(n_rows / bm), (int)N, K, (int)bm,
@@ -933,8 +979,7 @@ void expert_gemm(torch::Tensor out, torch::Tensor a, torch::Tensor w,
                         tile_off.data_ptr<int>(), counts.data_ptr<int>(),
                         (int)E, (int)N, (int)K, (int)bm, n_rows,
                         act == 2 ? 1 : (act == 3 ? 2 : (act == 1 ? 3 : 0)),
-                        (float)limit, kind,
-                        cur_stream());
+                        (float)limit, rw, kind, cur_stream());
 }
 
 // ---- pre-norm layers, decay recurrences ----
@@ -1023,6 +1068,81 @@ void add_rmsnorm(torch::Tensor x, c10::optional<torch::Tensor> y,
                   ld2, (int)sg_off, (const float*)opt_ptr(norm_w), (float)eps,
                   h_out.has_value() ? h_out->data_ptr() : nullptr, T, (int)W,
                   kind, cur_stream());
+}
+
+// ---- hyper-connections ----
+
+void hyper_rmsnorm(torch::Tensor x, c10::optional<torch::Tensor> x_in,
+                   c10::optional<torch::Tensor> y,
+                   c10::optional<torch::Tensor> rows,
+                   c10::optional<torch::Tensor> padpos,
+                   c10::optional<torch::Tensor> wts, double wconst,
+                   c10::optional<torch::Tensor> y2,
+                   c10::optional<torch::Tensor> mix,
+                   c10::optional<torch::Tensor> out,
+                   c10::optional<torch::Tensor> in,
+                   c10::optional<torch::Tensor> norm_w, double eps,
+                   c10::optional<torch::Tensor> h_out, bool write) {
+  CHECK_GPU(x); CHECK_CONTIG(x); CHECK_F32(x);
+  TORCH_CHECK(x.dim() == 3, "x must be [T, streams, W]");
+  const long T = x.size(0), S = x.size(1), W = x.size(2);
+  int kind = -1;
+  auto act = [&](const torch::Tensor& t, const char* what) {
+    CHECK_GPU(t); CHECK_CONTIG(t);
+    const int k = act_kind(t);
+    TORCH_CHECK(kind < 0 || kind == k, what, ": activation dtypes differ");
+    TORCH_CHECK(t.dim() == 2 && t.size(1) == W, what, " must be [*, W]");
+    kind = k;
+  };
+  if (x_in.has_value()) {
+    CHECK_GPU(*x_in); CHECK_F32(*x_in); CHECK_CONTIG(*x_in);
+    TORCH_CHECK(x_in->dim() == 2 && x_in->size(0) == T && x_in->size(1) == W,
+                "x_in must be [T, W]");
+  }
+  for (const auto& t : {y, y2, h_out}) {
+    if (!t.has_value()) continue;
+    act(*t, "row operand");
+    TORCH_CHECK(t->size(0) == T, "row operands must be [T, W]");
+  }
+  int k = 0;
+  if (rows.has_value()) {
+    act(*rows, "rows");
+    TORCH_CHECK(padpos.has_value(), "expert rows need padpos");
+    CHECK_GPU(*padpos); CHECK_I32(*padpos); CHECK_CONTIG(*padpos);
+    TORCH_CHECK(padpos->dim() == 2 && padpos->size(0) == T, "padpos shape");
+    if (wts.has_value()) {
+      CHECK_GPU(*wts); CHECK_F32(*wts); CHECK_CONTIG(*wts);
+      TORCH_CHECK(wts->sizes() == padpos->sizes(), "expert weights shape");
+    }
+    k = (int)padpos->size(1);
+  }
+  TORCH_CHECK(mix.has_value() == out.has_value(), "an update needs mix and out");
+  TORCH_CHECK(mix.has_value() || !(y.has_value() || rows.has_value() ||
+                                   y2.has_value()),
+              "a result needs mix and out");
+  TORCH_CHECK(!h_out.has_value() || (in.has_value() && norm_w.has_value()),
+              "a read needs its weights and the norm weight");
+  const float* mp = opt_f32(mix, S * S, "mix");
+  const float* op = opt_f32(out, S, "out");
+  const float* ip = opt_f32(in, S, "in");
+  const float* np = opt_f32(norm_w, W, "norm weight");
+  TORCH_CHECK(
+      mix_hyper_rmsnorm(
+          x.data_ptr<float>(), (const float*)opt_ptr(x_in), opt_ptr(y),
+          opt_ptr(rows), rows.has_value() ? (const int*)opt_ptr(padpos) : nullptr,
+          rows.has_value() ? (const float*)opt_ptr(wts) : nullptr,
+          (float)wconst, k, opt_ptr(y2), mp, op, ip, np, (float)eps,
+          h_out.has_value() ? h_out->data_ptr() : nullptr,
+          write && mix.has_value() ? 1 : 0, T, (int)S, (int)W,
+          kind < 0 ? 1 : kind, cur_stream()),
+      "hyper_rmsnorm: ", S, " streams of width ", W, " need ",
+      mix_hyper_lds((int)S, (int)W), " bytes of LDS, more than a block has");
+}
+
+void relu_sq(torch::Tensor z) {
+  CHECK_GPU(z); CHECK_CONTIG(z);
+  TORCH_CHECK((size_t)z.data_ptr() % 16 == 0, "16-byte alignment");
+  mix_relu_sq(z.data_ptr(), z.numel(), act_kind(z), cur_stream());
 }
 
 void glu_mul(torch::Tensor out, torch::Tensor proj, long gate_off, long up_off,
@@ -1144,7 +1264,7 @@ void rotary_sections(torch::Tensor out, torch::Tensor proj, long q_off,
 void latent_prep(torch::Tensor proj, long off, torch::Tensor norm_w, double eps,
                  torch::Tensor cos_sin, torch::Tensor cache,
                  torch::Tensor rows, torch::Tensor q, long q_off,
-                 torch::Tensor qa) {
+                 torch::Tensor qa, bool adjacent) {
   CHECK_GPU(proj); CHECK_GPU(cache); CHECK_CONTIG(cache); CHECK_GPU(qa);
   CHECK_CONTIG(qa); CHECK_GPU(q); CHECK_I64(rows); CHECK_CONTIG(rows);
   CHECK_GPU(norm_w); CHECK_F32(norm_w); CHECK_CONTIG(norm_w);
@@ -1166,9 +1286,9 @@ void latent_prep(torch::Tensor proj, long off, torch::Tensor norm_w, double eps,
   const char* qp = (const char*)q.data_ptr() + q_off * q.element_size();
   mix_latent_prep(cache.data_ptr(), rows.data_ptr<long>(), proj.data_ptr(),
                   proj.stride(0), (int)off, norm_w.data_ptr<float>(),
-                  (float)eps, cos_sin.data_ptr<float>(), (int)R, (int)rd, qp,
-                  q.stride(0), q.stride(1), qa.data_ptr(), T, (int)H,
-                  act_kind(proj), cur_stream());
+                  (float)eps, cos_sin.data_ptr<float>(), (int)R, (int)rd,
+                  adjacent ? 1 : 0, qp, q.stride(0), q.stride(1),
+                  qa.data_ptr(), T, (int)H, act_kind(proj), cur_stream());
 }
 
 void rope_table(torch::Tensor out, torch::Tensor pos, torch::Tensor inv_freq,
@@ -1295,6 +1415,13 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("proj2"), py::arg("sg_off"), py::arg("norm_w"), py::arg("eps"),
         py::arg("h_out"), py::arg("x_in") = c10::nullopt,
         py::arg("extra") = c10::nullopt, py::arg("wconst") = 0.0);
+  m.def("hyper_rmsnorm", &hyper_rmsnorm,
+        "streams X <- mix^T X + out y; h = rmsnorm(in . X) * w",
+        py::arg("x"), py::arg("x_in"), py::arg("y"), py::arg("rows"),
+        py::arg("padpos"), py::arg("wts"), py::arg("wconst"), py::arg("y2"),
+        py::arg("mix"), py::arg("out"), py::arg("in_w"), py::arg("norm_w"),
+        py::arg("eps"), py::arg("h_out"), py::arg("write") = true);
+  m.def("relu_sq", &relu_sq, "max(z, 0)^2 in place");
   m.def("glu_mul", &glu_mul, "act(gate) * up: tanh-GELU, silu or clamped unit");
   m.def("moe_route_softmax", &moe_route_softmax,
         "softmax router: correction, group-limited choice, identity experts");
@@ -1304,7 +1431,10 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("rotary_sections", &rotary_sections,
         "fp32 q, k, v sections, q and k rotated on a prefix of every head");
   m.def("latent_prep", &latent_prep,
-        "normed latent | rotated key part into cache rows, rotated query parts");
+        "normed latent | rotated key part into cache rows, rotated query parts",
+        py::arg("proj"), py::arg("off"), py::arg("norm_w"), py::arg("eps"),
+        py::arg("cos_sin"), py::arg("cache"), py::arg("rows"), py::arg("q"),
+        py::arg("q_off"), py::arg("qa"), py::arg("adjacent") = false);
   m.def("rope_table", &rope_table, "cos | sin rows of the step's positions");
   m.def("moe_dispatch_table", &moe_dispatch_table,
         "token ids -> padded per-expert segments of their table rows");
@@ -1322,7 +1452,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("v_cache"), py::arg("v_first") = c10::nullopt,
         py::arg("v_first_off") = 0, py::arg("v_lambda") = c10::nullopt);
   m.def("local_attention", &local_attention,
-        "chunked/windowed paged attention with per-head output gate",
+        "chunked/windowed paged attention with an output gate and a sink",
         py::arg("out"), py::arg("out_off"), py::arg("q"), py::arg("k_cache"),
         py::arg("v_cache"), py::arg("bt"), py::arg("seq_lens"),
         py::arg("qlocs"), py::arg("token_seq"), py::arg("scale"),
@@ -1331,7 +1461,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("tile_seq") = c10::nullopt, py::arg("tile_q0") = c10::nullopt,
         py::arg("prefill_rows") = 0, py::arg("bias_r1") = c10::nullopt,
         py::arg("bias_r2") = c10::nullopt, py::arg("sink") = false,
-        py::arg("keep_first") = 0);
+        py::arg("keep_first") = 0, py::arg("gate_n") = 1,
+        py::arg("sink_w") = c10::nullopt);
   m.def("delta_prep", &delta_prep, "delta-rule inputs: filters, norms, gates",
         py::arg("qn"), py::arg("kn"), py::arg("v"), py::arg("decay"),
         py::arg("beta"), py::arg("proj"), py::arg("q_off"), py::arg("k_off"),
@@ -1363,14 +1494,20 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "layer-scaled parallel residual (second branch dense or gathered "
         "expert rows) + Dynamic-Tanh norm of the result");
   m.def("moe_route", &moe_route,
-        "sigmoid router with group-limited choice and normalised weights");
+        "sigmoid router with group-limited choice; the weights are the scores, "
+        "normalised or as they are",
+        py::arg("idx"), py::arg("wts"), py::arg("logits"), py::arg("groups"),
+        py::arg("keep"), py::arg("rank"), py::arg("renorm") = true);
   m.def("moe_dispatch", &moe_dispatch,
-        "(token, choice) pairs -> padded per-expert segments");
+        "(token, choice) pairs -> padded per-expert segments (and row weights)",
+        py::arg("row_tok"), py::arg("tile_off"), py::arg("counts"),
+        py::arg("padpos"), py::arg("idx"), py::arg("bm"),
+        py::arg("wts") = c10::nullopt, py::arg("row_w") = c10::nullopt);
   m.def("expert_gemm", &expert_gemm,
         "GEMM over padded per-expert segments (matrix cores for bf16 with "
         "64-aligned sizes, plain tiles otherwise)",
         py::arg("out"), py::arg("a"), py::arg("w"), py::arg("row_tok"),
         py::arg("tile_off"), py::arg("counts"), py::arg("act"), py::arg("bm"),
-        py::arg("limit") = 0.0);
+        py::arg("limit") = 0.0, py::arg("row_w") = c10::nullopt);
   m.def("softcap", &softcap, "cap * tanh(z / cap), fp32 out");
 }

@@ -5,14 +5,17 @@
 //                  layer without experts and the final norm.
 //   moe_route      sigmoid scores, group-limited choice (a group is worth the
 //                  sum of its `rank` largest scores, the `keep` best groups
-//                  stay), the `top` best experts and their normalised weights
+//                  stay), the `top` best experts and their weights (the
+//                  scores, normalised or as they are)
 //   moe_dispatch   (token, choice) pairs -> per-expert segments padded to the
 //                  GEMM tile height: row -> token table, segment starts,
-//                  counts, pair -> row table. LDS counters; one workgroup,
-//                  or three launches over runs of pairs
+//                  counts, pair -> row table, optionally the weight of every
+//                  row. LDS counters; one workgroup, or three launches over
+//                  runs of pairs
 //   expert_gemm    plain tiled GEMM over those segments for shapes or types
 //                  the matrix-core kernel (grouped_gemm.hip) does not take:
-//                  fp32 FMA, optional squared-ReLU epilogue
+//                  fp32 FMA, optional squared-ReLU or gated epilogue, rows
+//                  optionally weighted before it
 //   softcap        c * tanh(z / c) in fp32
 // The stream x, norm parameters, layer scales, router scores and weights are
 // fp32; `A` is the activation type (u16 = bf16 bits, or float).
@@ -99,7 +102,7 @@ __device__ __forceinline__ bool before(float va, int ia, float vb, int ib) {
 __global__ void __launch_bounds__(256) moe_route_kernel(
     int* __restrict__ idx, float* __restrict__ wts,
     const float* __restrict__ logits, long T, int E, int top, int G, int keep,
-    int rank) {
+    int rank, int renorm) {
   extern __shared__ float sm[];
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   float* sc = sm + wid * (E + G);
@@ -188,6 +191,7 @@ __global__ void __launch_bounds__(256) moe_route_kernel(
       wts[t * top + j] = s;
     }
   }
+  if (!renorm) return;
   __syncthreads();
   if (valid) {
     const float inv = 1.f / (total + 1e-20f);
@@ -197,18 +201,20 @@ __global__ void __launch_bounds__(256) moe_route_kernel(
 
 extern "C" void mix_moe_route(int* idx, float* wts, const float* logits, long T,
                               int E, int top, int G, int keep, int rank,
-                              hipStream_t s) {
+                              int renorm, hipStream_t s) {
   if (T == 0) return;
   const size_t smem = (size_t)4 * (E + G) * sizeof(float);
   hipLaunchKernelGGL(moe_route_kernel, dim3((unsigned)((T + 3) / 4)), dim3(256),
-                     smem, s, idx, wts, logits, T, E, top, G, keep, rank);
+                     smem, s, idx, wts, logits, T, E, top, G, keep, rank,
+                     renorm);
 }
 
 // ---- moe_dispatch ----------------------------------------------------------
 // The place of a pair inside its expert's segment comes from an LDS counter, so
 // it depends on timing; a row's result does not depend on its place, and every
 // pair finds its row through padpos. With `ids`, idx is a table [vocab, k] and
-// pair i uses its row ids[i / k].
+// pair i uses its row ids[i / k]. With `row_w`, row r of pair i also gets
+// row_w[r] = wts[i] (0 for padding rows).
 __device__ __forceinline__ int pair_expert(const int* __restrict__ idx,
                                            const long* __restrict__ ids, int i,
                                            int t, int k) {
@@ -220,7 +226,8 @@ __global__ void __launch_bounds__(1024) moe_dispatch_kernel(
     int* __restrict__ row_tok, int* __restrict__ tile_off,
     int* __restrict__ counts, int* __restrict__ padpos,
     const int* __restrict__ idx, const long* __restrict__ ids, int n_pairs,
-    int k, int E, int bm, long n_rows) {
+    int k, int E, int bm, long n_rows, const float* __restrict__ wts,
+    float* __restrict__ row_w) {
   extern __shared__ int smi[];
   int* cnt = smi;          // [E] pairs per expert, then a running cursor
   int* start = smi + E;    // [E + 1] first padded row of each segment
@@ -229,7 +236,10 @@ __global__ void __launch_bounds__(1024) moe_dispatch_kernel(
   __syncthreads();
   for (int i = tid; i < n_pairs; i += 1024)
     atomicAdd(&cnt[pair_expert(idx, ids, i, i / k, k)], 1);
-  for (long i = tid; i < n_rows; i += 1024) row_tok[i] = -1;
+  for (long i = tid; i < n_rows; i += 1024) {
+    row_tok[i] = -1;
+    if (row_w) row_w[i] = 0.f;
+  }
   __syncthreads();
   if (tid == 0) {
     int off = 0;
@@ -252,6 +262,7 @@ __global__ void __launch_bounds__(1024) moe_dispatch_kernel(
     const int r = start[e] + atomicAdd(&cnt[e], 1);
     row_tok[r] = t;
     padpos[i] = r;
+    if (row_w) row_w[r] = wts[i];
   }
 }
 
@@ -263,7 +274,7 @@ __global__ void __launch_bounds__(1024) moe_dispatch_kernel(
 __global__ void __launch_bounds__(256) moe_count_kernel(
     int* __restrict__ hist, int* __restrict__ row_tok,
     const int* __restrict__ idx, const long* __restrict__ ids, int n_pairs,
-    int k, int E, long n_rows) {
+    int k, int E, long n_rows, float* __restrict__ row_w) {
   extern __shared__ int smi[];
   for (int e = threadIdx.x; e < E; e += 256) smi[e] = 0;
   __syncthreads();
@@ -277,8 +288,10 @@ __global__ void __launch_bounds__(256) moe_count_kernel(
   for (int n = 0; n < DCH / 256; ++n)
     if (ex[n] >= 0) atomicAdd(&smi[ex[n]], 1);
   for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < n_rows;
-       i += (long)gridDim.x * 256)
+       i += (long)gridDim.x * 256) {
     row_tok[i] = -1;
+    if (row_w) row_w[i] = 0.f;
+  }
   __syncthreads();
   for (int e = threadIdx.x; e < E; e += 256)
     hist[(long)blockIdx.x * E + e] = smi[e];
@@ -314,7 +327,8 @@ __global__ void __launch_bounds__(256) moe_place_kernel(
     int* __restrict__ row_tok, int* __restrict__ padpos,
     const int* __restrict__ hist, const int* __restrict__ tile_off,
     const int* __restrict__ idx, const long* __restrict__ ids, int n_pairs,
-    int k, int E, int bm) {
+    int k, int E, int bm, const float* __restrict__ wts,
+    float* __restrict__ row_w) {
   extern __shared__ int smi[];  // [E] next row of each segment
   for (int e = threadIdx.x; e < E; e += 256)
     smi[e] = tile_off[e] * bm + hist[(long)blockIdx.x * E + e];
@@ -332,6 +346,7 @@ __global__ void __launch_bounds__(256) moe_place_kernel(
     const int r = atomicAdd(&smi[ex[n]], 1);
     row_tok[r] = i / k;
     padpos[i] = r;
+    if (row_w) row_w[r] = wts[i];
   }
 }
 
@@ -343,23 +358,24 @@ extern "C" long mix_moe_dispatch_scratch(long n_pairs, int E) {
 extern "C" void mix_moe_dispatch(int* row_tok, int* tile_off, int* counts,
                                  int* padpos, const int* idx, const long* ids,
                                  long n_pairs, int k, int E, int bm,
-                                 long n_rows, int* scratch, hipStream_t s) {
+                                 long n_rows, int* scratch, const float* wts,
+                                 float* row_w, hipStream_t s) {
   if (!scratch) {
     const size_t smem = (size_t)(2 * E + 1) * sizeof(int);
     hipLaunchKernelGGL(moe_dispatch_kernel, dim3(1), dim3(1024), smem, s,
                        row_tok, tile_off, counts, padpos, idx, ids,
-                       (int)n_pairs, k, E, bm, n_rows);
+                       (int)n_pairs, k, E, bm, n_rows, wts, row_w);
     return;
   }
   const int runs = (int)((n_pairs + DCH - 1) / DCH);
   const size_t smem = (size_t)E * sizeof(int);
   hipLaunchKernelGGL(moe_count_kernel, dim3(runs), dim3(256), smem, s, scratch,
-                     row_tok, idx, ids, (int)n_pairs, k, E, n_rows);
+                     row_tok, idx, ids, (int)n_pairs, k, E, n_rows, row_w);
   hipLaunchKernelGGL(moe_offsets_kernel, dim3(1), dim3(1024), smem, s, scratch,
                      tile_off, counts, runs, E, bm);
   hipLaunchKernelGGL(moe_place_kernel, dim3(runs), dim3(256), smem, s, row_tok,
                      padpos, scratch, tile_off, idx, ids, (int)n_pairs, k, E,
-                     bm);
+                     bm, wts, row_w);
 }
 
 // ---- expert_gemm (plain) ---------------------------------------------------
@@ -368,13 +384,14 @@ extern "C" void mix_moe_dispatch(int* row_tok, int* tile_off, int* counts,
 // 16 at a time through LDS. Rows past a segment's live count are not stored.
 // act 1: relu(x)^2. act 2: w holds N gate rows then N up rows per expert and
 // out[r, n] = g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up).
-// act 3: the same two row blocks, out[r, n] = silu(g) u.
+// act 3: the same two row blocks, out[r, n] = silu(g) u. With row_w the products
+// of row r are multiplied by row_w[r] before the activation.
 template <typename A>
 __global__ void __launch_bounds__(256) expert_gemm_plain_kernel(
     A* __restrict__ out, const A* __restrict__ a, const A* __restrict__ w,
     const int* __restrict__ row_tok, const int* __restrict__ tile_off,
     const int* __restrict__ counts, int E, int N, int K, int bm, int act,
-    float limit) {
+    float limit, const float* __restrict__ row_w) {
   __shared__ float As[16][65];
   __shared__ float Bs[16][65];
   __shared__ float Us[16][65];
@@ -444,11 +461,13 @@ __global__ void __launch_bounds__(256) expert_gemm_plain_kernel(
   for (int i = 0; i < 4; ++i) {
     const int r = ty * 4 + i;
     if (r >= live) continue;
+    const float rw = row_w ? row_w[seg + r] : 1.f;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
       if (n >= N) continue;
-      float v = acc[i][j];
+      float v = acc[i][j] * rw;
+      accu[i][j] *= rw;
       if (act == 1) {
         v = v > 0.f ? v : 0.f;
         v *= v;
@@ -468,18 +487,19 @@ extern "C" void mix_expert_gemm_plain(void* out, const void* a, const void* w,
                                       const int* row_tok, const int* tile_off,
                                       const int* counts, int E, int N, int K,
                                       int bm, long n_rows, int act, float limit,
-                                      int f32, hipStream_t s) {
+                                      const float* row_w, int f32,
+                                      hipStream_t s) {
   const long tiles = n_rows / 64;
   if (tiles == 0) return;
   const dim3 grid((unsigned)tiles, (unsigned)((N + 63) / 64));
   if (f32)
     hipLaunchKernelGGL(expert_gemm_plain_kernel<float>, grid, dim3(256), 0, s,
                        (float*)out, (const float*)a, (const float*)w, row_tok,
-                       tile_off, counts, E, N, K, bm, act, limit);
+                       tile_off, counts, E, N, K, bm, act, limit, row_w);
   else
     hipLaunchKernelGGL(expert_gemm_plain_kernel<u16>, grid, dim3(256), 0, s,
                        (u16*)out, (const u16*)a, (const u16*)w, row_tok,
-                       tile_off, counts, E, N, K, bm, act, limit);
+                       tile_off, counts, E, N, K, bm, act, limit, row_w);
 }
 
 // ---- softcap ---------------------------------------------------------------

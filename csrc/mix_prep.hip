@@ -10,7 +10,8 @@
 //   sigmoid_gate_mul  v *= sigmoid(gate section), elementwise
 //   latent_prep       latent attention with a rotated key part: normed latent
 //                     and rotated key part of every token into its cache row,
-//                     rotated query parts behind the folded queries
+//                     rotated query parts behind the folded queries; pairs
+//                     (i, i + rd/2) or neighbours (2i, 2i + 1)
 //   rope_table        cos | sin rows of the positions of a step
 // One 256-thread block a token (and section); fp32 math.
 #include "mix_common.h"
@@ -117,7 +118,7 @@ template <typename A>
 __global__ void __launch_bounds__(256) latent_prep_kernel(
     A* __restrict__ cache, const long* __restrict__ rows,
     const A* __restrict__ proj, long ld, int off, const float* __restrict__ w,
-    float eps, const float* __restrict__ cos_sin, int R, int rd,
+    float eps, const float* __restrict__ cos_sin, int R, int rd, int adjacent,
     const A* __restrict__ q, long sqt, long sqh, A* __restrict__ qa, int H) {
   __shared__ float red[4];
   const long t = blockIdx.x;
@@ -138,16 +139,18 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(
     const int u = e / half, i = e - u * half;
     const A* in = u < H ? q + t * sqt + u * sqh : src + R;
     A* o = u < H ? qa + (t * H + u) * (long)(R + rd) + R : dst + R;
-    const float a = ldf<A>(in + i), b = ldf<A>(in + half + i);
+    const int ia = adjacent ? 2 * i : i, ib = adjacent ? 2 * i + 1 : half + i;
+    const float a = ldf<A>(in + ia), b = ldf<A>(in + ib);
     const float c = cs[i], sn = cs[half + i];
-    stf<A>(o + i, a * c - b * sn);
-    stf<A>(o + half + i, b * c + a * sn);
+    stf<A>(o + ia, a * c - b * sn);
+    stf<A>(o + ib, b * c + a * sn);
   }
 }
 
 // bf16, 16 bytes a lane: the first wave of a workgroup norms the latent (kept
 // in registers up to 512 wide), the other two turn 8 pairs a lane. Needs R,
 // half the rotated part and every offset and stride to be multiples of 8.
+template <bool ADJ>
 __global__ void __launch_bounds__(192) latent_prep_vec_kernel(
     u16* __restrict__ cache, const long* __restrict__ rows,
     const u16* __restrict__ proj, long ld, int off, const float* __restrict__ w,
@@ -185,9 +188,25 @@ __global__ void __launch_bounds__(192) latent_prep_vec_kernel(
     const int u = j / per, i = (j - u * per) * 8;
     const u16* in = u < H ? q + t * sqt + u * sqh : src + R;
     u16* o = u < H ? qa + (t * H + u) * (long)(R + rd) + R : dst + R;
+    // the 8 pairs lie in two vectors: first and second members (halves), or
+    // pairs 0..3 and pairs 4..7 (neighbours)
+    const int p0 = ADJ ? 2 * i : i, p1 = ADJ ? 2 * i + 8 : half + i;
     float a[8], b[8];
-    bf8_to_f32(*(const u16x8*)(in + i), a);
-    bf8_to_f32(*(const u16x8*)(in + half + i), b);
+    bf8_to_f32(*(const u16x8*)(in + p0), a);
+    bf8_to_f32(*(const u16x8*)(in + p1), b);
+    if (ADJ) {
+      float x[16];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        x[e] = a[e];
+        x[8 + e] = b[e];
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        a[e] = x[2 * e];
+        b[e] = x[2 * e + 1];
+      }
+    }
     u16x8 oa, ob;
 #pragma unroll
     for (int h = 0; h < 2; ++h) {
@@ -196,40 +215,60 @@ __global__ void __launch_bounds__(192) latent_prep_vec_kernel(
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int k = 4 * h + e;
-        oa[k] = f2bf(a[k] * c[e] - b[k] * s[e]);
-        ob[k] = f2bf(b[k] * c[e] + a[k] * s[e]);
+        const u16 ya = f2bf(a[k] * c[e] - b[k] * s[e]);
+        const u16 yb = f2bf(b[k] * c[e] + a[k] * s[e]);
+        if (ADJ) {
+          if (h == 0) {
+            oa[2 * e] = ya;
+            oa[2 * e + 1] = yb;
+          } else {
+            ob[2 * e] = ya;
+            ob[2 * e + 1] = yb;
+          }
+        } else {
+          oa[k] = ya;
+          ob[k] = yb;
+        }
       }
     }
-    *(u16x8*)(o + i) = oa;
-    *(u16x8*)(o + half + i) = ob;
+    *(u16x8*)(o + p0) = oa;
+    *(u16x8*)(o + p1) = ob;
   }
 }
 
 extern "C" void mix_latent_prep(void* cache, const long* rows, const void* proj,
                                 long ld, int off, const float* w, float eps,
                                 const float* cos_sin, int R, int rd,
-                                const void* q, long sqt, long sqh, void* qa,
-                                long T, int H, int f32, hipStream_t s) {
+                                int adjacent, const void* q, long sqt,
+                                long sqh, void* qa, long T, int H, int f32,
+                                hipStream_t s) {
   if (T == 0) return;
   if (!f32 && R % 8 == 0 && rd % 16 == 0 && off % 8 == 0 && ld % 8 == 0 &&
       sqt % 8 == 0 && sqh % 8 == 0 && (size_t)q % 16 == 0 &&
       (size_t)proj % 16 == 0 && (size_t)qa % 16 == 0 &&
       (size_t)cache % 16 == 0) {
-    hipLaunchKernelGGL(latent_prep_vec_kernel, dim3((unsigned)T), dim3(192), 0,
-                       s, (u16*)cache, rows, (const u16*)proj, ld, off, w, eps,
-                       cos_sin, R, rd, (const u16*)q, sqt, sqh, (u16*)qa, H);
+    if (adjacent)
+      hipLaunchKernelGGL(latent_prep_vec_kernel<true>, dim3((unsigned)T),
+                         dim3(192), 0, s, (u16*)cache, rows, (const u16*)proj,
+                         ld, off, w, eps, cos_sin, R, rd, (const u16*)q, sqt,
+                         sqh, (u16*)qa, H);
+    else
+      hipLaunchKernelGGL(latent_prep_vec_kernel<false>, dim3((unsigned)T),
+                         dim3(192), 0, s, (u16*)cache, rows, (const u16*)proj,
+                         ld, off, w, eps, cos_sin, R, rd, (const u16*)q, sqt,
+                         sqh, (u16*)qa, H);
     return;
   }
   if (f32)
     hipLaunchKernelGGL(latent_prep_kernel<float>, dim3((unsigned)T), dim3(256),
                        0, s, (float*)cache, rows, (const float*)proj, ld, off,
-                       w, eps, cos_sin, R, rd, (const float*)q, sqt, sqh,
-                       (float*)qa, H);
+                       w, eps, cos_sin, R, rd, adjacent, (const float*)q, sqt,
+                       sqh, (float*)qa, H);
   else
     hipLaunchKernelGGL(latent_prep_kernel<u16>, dim3((unsigned)T), dim3(256),
                        0, s, (u16*)cache, rows, (const u16*)proj, ld, off, w,
-                       eps, cos_sin, R, rd, (const u16*)q, sqt, sqh, (u16*)qa,
-                       H);
+                       eps, cos_sin, R, rd, adjacent, (const u16*)q, sqt, sqh,
+                       (u16*)qa, H);
 }
 
 // out[t]: amp * cos(pos f_i) [half] | amp * sin(pos f_i) [half], fp32 angles

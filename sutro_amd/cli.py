@@ -218,7 +218,7 @@ def generate(model: str, prompts, max_tokens: int, temperature: float,
         from .build import ensure_built
 
         layer_list = cfg.spec.arch in ("vodinex", "ruludra", "vukotar",
-                                      "nosalorn", "vanulorn")
+                                      "nosalorn", "vanulorn", "tubepel")
         ensure_built(["_C", "_C_mix"] if layer_list else ["_C"])
     eng = LLMEngine(cfg)
     outs = eng.generate(list(prompts), sampling=SamplingParams(

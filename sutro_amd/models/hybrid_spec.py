@@ -3,10 +3,10 @@ mixer and feed-forward, so attention layers, recurrent layers and layers that
 run both side by side can be ordered freely.
 
 A spec is built from a checkpoint's ``config.json`` (see :func:`vodinex_spec`,
-:func:`ruludra_spec`, :func:`vukotar_spec`, :func:`nosalorn_spec` and
-:func:`vanulorn_spec`) or directly in code (tests, benchmarks). Nothing here
-fixes a size: widths, head counts, mask sizes, filter lengths and the order of
-layers all come from the config.
+:func:`ruludra_spec`, :func:`vukotar_spec`, :func:`nosalorn_spec`,
+:func:`vanulorn_spec` and :func:`tubepel_spec`) or directly in code (tests,
+benchmarks). Nothing here fixes a size: widths, head counts, mask sizes, filter
+lengths and the order of layers all come from the config.
 """
 
 from __future__ import annotations
@@ -46,10 +46,13 @@ class AttnMixerSpec:
     window: int = 0
     qk_norm: bool = True
     bias: bool = True        # q/k/v/o projections carry biases
-    out_gate: bool = True    # one sigmoid gate per head on the attention output
+    out_gate: bool = True    # sigmoid gate on the attention output
+    gate_elements: bool = False  # one gate per element instead of one per head
     # a silent sink: a key of score 0 without a value takes part in the
     # normalisation, p_j = exp(s_j) / (1 + sum_j exp(s_j))
     sink: bool = False
+    # the sink's score is a learned number per head instead of 0
+    sink_learned: bool = False
     keep_first: int = 0
     rot_scaling: Optional[Tuple[float, float, float, float]] = None
     v_mix: bool = False
@@ -120,7 +123,9 @@ class LatentAttnMixerSpec:
     ``rot_dim``: that many further query dimensions per head are rotated and
     meet one rotated key part shared by all heads (projected beside the
     latent, not normed, cached beside it); 0 = no positions. ``rot_base`` and
-    ``rot_scaling`` as in :class:`AttnMixerSpec`."""
+    ``rot_scaling`` as in :class:`AttnMixerSpec`. ``rot_adjacent``: dimensions
+    2i and 2i + 1 of the rotated part turn together instead of i and i +
+    rot_dim / 2."""
 
     heads: int
     dim: int
@@ -134,6 +139,7 @@ class LatentAttnMixerSpec:
     rot_base: float = 10000.0
     rot_scaling: Optional[Tuple[float, float, float, float]] = None
     out_gate: bool = True
+    rot_adjacent: bool = False
 
 
 @dataclass(frozen=True)
@@ -201,7 +207,9 @@ class RoutedExpertsSpec:
     feed-forwards of inner width `ff`, of which a token uses `top`.
 
     ``router``: "sigmoid" scores every expert by the sigmoid of its logit and
-    weights the chosen ones by score / (sum of chosen scores + 1e-20).
+    weights the chosen ones by score / (sum of chosen scores + 1e-20), or by
+    the score itself (``renorm`` off). ``weigh_input``: the weight multiplies
+    the input of an expert instead of its result.
     ``groups`` / ``keep``: the experts form `groups` equal runs of neighbours;
     a run is worth the sum of its `group_rank` largest scores and only experts
     of the `keep` best runs can be chosen (groups = keep = 1: no restriction).
@@ -240,6 +248,8 @@ class RoutedExpertsSpec:
     shared_limit: float = 0.0
     shared_gate: bool = True
     vocab: int = 0
+    renorm: bool = True
+    weigh_input: bool = False
 
 
 @dataclass(frozen=True)
@@ -247,6 +257,8 @@ class HybridLayerSpec:
     kind: str                # the config's layer type
     mixer: MixerSpec
     ff: int = 0              # 0 = the layer has no (dense) feed-forward
+    # how a dense feed-forward looks where designs differ: "swiglu" =
+    # down(silu(gate h) (up h)), "relu2" = down(max(up h, 0)^2)
     ff_kind: str = "dense"
     moe: Optional[RoutedExpertsSpec] = None
     # index of the layer whose parameters this layer uses (its cache is its
@@ -276,9 +288,14 @@ class HybridSpec:
     embed_scale: float = 1.0     # multiplies the token row
     logit_softcap: float = 0.0   # c * tanh(logits / c); 0 = none
     # (start, stop, times): the layers of range(start, stop) are gone through
-    # `times` times, sharing weights but not cache or state; the embedding
-    # output re-enters the stream whenever a further pass begins
+    # `times` times, sharing weights but not cache or state; with
+    # `loop_reenter` the embedding output re-enters the stream whenever a
+    # further pass begins
     loop: Optional[Tuple[int, int, int]] = None
+    loop_reenter: bool = True
+    # hyper-connections: that many residual streams, mixed and read through
+    # learned weights around every sublayer; 0 = one plain residual
+    streams: int = 0
     # what is added to a stored norm weight of the pre-norm layers (1.0 where
     # checkpoints keep the gain's distance from one)
     norm_offset: float = 0.0
@@ -323,7 +340,7 @@ class HybridSpec:
             return self._sandwich_param_count()
         if self.arch == "vukotar":
             return self._parallel_param_count(active=False)
-        if self.arch in ("nosalorn", "vanulorn"):
+        if self.arch in ("nosalorn", "vanulorn", "tubepel"):
             return self._prenorm_param_count(active=False)
         for layer in self.layers:
             m = layer.mixer
@@ -396,13 +413,21 @@ class HybridSpec:
             layer = self.layers[i]
             m = layer.mixer
             n += h
+            if self.streams:
+                n += (2 if layer.ff or layer.moe else 1) \
+                    * self.streams * (self.streams + 2)
             if isinstance(m, AttnMixerSpec):
                 cols = m.heads * m.dim + m.kv_heads * (m.dim + m.vdim)
-                n += (h + 1) * cols + m.heads * m.vdim * h + int(m.v_mix)
+                n += (h + int(m.bias)) * cols + m.heads * m.vdim * h
+                n += int(m.v_mix) + (m.heads if m.sink_learned else 0)
+                if m.out_gate:
+                    n += h * m.heads * (m.vdim if m.gate_elements else 1)
             elif isinstance(m, LatentAttnMixerSpec):
-                H, R = m.heads, m.kv_rank
-                n += h * (H * (m.dim + m.rot_dim) + R + m.rot_dim) + R
+                H, R, qc = m.heads, m.kv_rank, m.heads * (m.dim + m.rot_dim)
+                n += m.q_rank * (h + 1 + qc) if m.q_rank else h * qc
+                n += h * (R + m.rot_dim) + R
                 n += H * (m.dim + m.vdim) * R + H * m.vdim * h
+                n += h * H * m.vdim if m.out_gate else 0
             elif isinstance(m, DecayAttnMixerSpec):
                 hv = m.heads * m.vdim
                 n += h * (2 * m.heads * m.dim + 2 * hv) + hv * h
@@ -417,12 +442,12 @@ class HybridSpec:
                 n += (inner + bc) * (m.conv + 1) + 3 * m.heads + inner
                 n += inner * h
             if layer.ff:
-                n += h + 3 * h * layer.ff
+                n += h + (2 if layer.ff_kind == "relu2" else 3) * h * layer.ff
             if layer.moe:
                 e = layer.moe
                 n += h
                 if e.router != "table":
-                    n += (e.experts + e.identity) * (h + 1)
+                    n += (e.experts + e.identity) * (h + int(e.correction))
                 n += (min(e.top, e.experts) if active else e.experts) \
                     * 3 * h * e.ff
                 if e.shared_ff:
@@ -432,7 +457,7 @@ class HybridSpec:
     def active_param_count(self) -> int:
         if self.arch == "vukotar":
             return self._parallel_param_count(active=True)
-        if self.arch in ("nosalorn", "vanulorn"):
+        if self.arch in ("nosalorn", "vanulorn", "tubepel"):
             return self._prenorm_param_count(active=True)
         return self.param_count()
 
@@ -443,6 +468,18 @@ def _rot_scaling(rot: dict) -> Optional[Tuple[float, float, float, float]]:
         return None
     return (float(sc["factor"]), float(sc["original"]), float(sc["fast"]),
             float(sc["slow"]))
+
+
+def _loop(config: dict, n_layers: int) -> Optional[Tuple[int, int, int]]:
+    """(start, stop, times) of a config's loop; None where nothing repeats."""
+    lp = config.get("loop")
+    if not lp or int(lp["times"]) == 1 or int(lp["start"]) == int(lp["stop"]):
+        return None
+    loop = (int(lp["start"]), int(lp["stop"]), int(lp["times"]))
+    if not 0 <= loop[0] < loop[1] <= n_layers or loop[2] < 1:
+        raise ValueError("loop must name a run of layers and be passed at "
+                         "least once")
+    return loop
 
 
 def _delta_from_config(m: dict, ranks: Tuple[int, int]) -> DeltaMixerSpec:
@@ -805,13 +842,6 @@ def vanulorn_spec(config: dict, name: str = "vanulorn",
                 raise ValueError(f"unknown feed-forward kind {fk!r}")
         layers.append(HybridLayerSpec(kind=kind, mixer=mixer, ff=ff,
                                       ff_kind="swiglu", moe=moe))
-    lp = config.get("loop")
-    loop = None
-    if lp and int(lp["times"]) != 1 and int(lp["start"]) != int(lp["stop"]):
-        loop = (int(lp["start"]), int(lp["stop"]), int(lp["times"]))
-        if not 0 <= loop[0] < loop[1] <= len(layers) or loop[2] < 1:
-            raise ValueError("loop must name a run of layers and be passed at "
-                             "least once")
     emb = config.get("embedding") or {}
     big = emb.get("bigram")
     return HybridSpec(
@@ -822,7 +852,87 @@ def vanulorn_spec(config: dict, name: str = "vanulorn",
         checkpoint_dir=checkpoint_dir,
         bigram=(int(big["buckets"]), int(big["mul_prev"]),
                 int(big["mul_cur"])) if big else None,
-        embed_scale=float(emb.get("scale", 1.0)), loop=loop, norm_offset=1.0,
+        embed_scale=float(emb.get("scale", 1.0)),
+        loop=_loop(config, len(layers)), norm_offset=1.0,
         tie_embeddings=True,
+        num_experts=max([(l.moe.experts if l.moe else 0) for l in layers]
+                        + [0]))
+
+
+def tubepel_spec(config: dict, name: str = "tubepel",
+                 checkpoint_dir: Optional[str] = None,
+                 tensor_shapes: Optional[dict] = None) -> HybridSpec:
+    """Build the spec of a Tubepel checkpoint from its ``config.json``: a list
+    of pre-norm layers (weighted RMS norms) over several residual streams
+    (hyper-connections), each with a rotary latent attention with a query
+    latent (two kinds, which differ in the pairing of the rotated dimensions)
+    or a windowed attention with kept first tokens, learned sinks and an
+    elementwise output gate, and an optional squared-ReLU or routed-experts
+    feed-forward (sigmoid scores that weigh the experts' input); a run of
+    layers that is passed several times; untied head. A latent's query rank is
+    `q_rank` of the mixer dict, or else the row count of ``<mixer>.dq`` in
+    ``tensor_shapes``."""
+    shapes = tensor_shapes or {}
+    layers = []
+    for i, lc in enumerate(config["layers"]):
+        kind = lc["type"]
+        m = lc["mixer"]
+        rot = m.get("rot") or {}
+        if kind in ("latent_attention", "latent_attention_2"):
+            q_rank = m.get("q_rank")
+            if q_rank is None:
+                q_rank = shapes[f"l{i}.mix.dq"][0]
+            mixer: MixerSpec = LatentAttnMixerSpec(
+                heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                q_rank=int(q_rank), kv_rank=int(m["kv_rank"]),
+                scale=float(m["scale"]), rot_dim=int(m.get("rot_dim", 0) or 0),
+                rot_base=float(rot.get("base", 10000.0)), out_gate=False,
+                rot_adjacent=kind == "latent_attention")
+            if int(rot.get("dims", mixer.rot_dim)) != mixer.rot_dim:
+                raise ValueError(f"layer {i}: the whole rotated part turns, so "
+                                 f"rot.dims must equal rot_dim")
+        elif kind == "attention":
+            mask = m.get("mask") or {}
+            mixer = AttnMixerSpec(
+                heads=int(m["heads"]), kv_heads=int(m["kv_heads"]),
+                dim=int(m["dim"]), vdim=int(m["vdim"]),
+                scale=float(m["scale"]), rot_dims=int(rot.get("dims", 0) or 0),
+                rot_base=float(rot.get("base", 10000.0)),
+                window=int(mask.get("size", 0) or 0),
+                keep_first=int(mask.get("keep_first", 0) or 0),
+                qk_norm=False, bias=False, out_gate=True, gate_elements=True,
+                sink=True, sink_learned=True)
+        else:
+            raise ValueError(f"unknown layer type {kind!r} in layer {i}")
+        mlp = lc.get("mlp")
+        ff, moe = 0, None
+        if mlp is not None:
+            fk = mlp.get("kind", "dense")
+            if fk == "dense":
+                ff = int(mlp["ff"])
+            elif fk == "moe":
+                r = mlp["router"]
+                moe = RoutedExpertsSpec(
+                    ff=int(mlp["expert"]["ff"]), experts=int(r["experts"]),
+                    top=int(r["top"]), router="sigmoid", act="silu_glu",
+                    shared_ff=int((mlp.get("shared") or {}).get("ff", 0) or 0),
+                    shared_gate=False, renorm=False, weigh_input=True)
+                if not 1 <= moe.top <= moe.experts:
+                    raise ValueError(f"layer {i}: a token uses 1..experts "
+                                     f"experts")
+            else:
+                raise ValueError(f"unknown feed-forward kind {fk!r}")
+        layers.append(HybridLayerSpec(kind=kind, mixer=mixer, ff=ff,
+                                      ff_kind="relu2", moe=moe))
+    streams = int(config["streams"])
+    if streams < 1:
+        raise ValueError("streams must be at least 1")
+    return HybridSpec(
+        name=name, arch="tubepel", hidden_size=int(config["width"]),
+        vocab_size=int(config["vocab"]), layers=tuple(layers),
+        norm_eps=float(config["norm"]["eps"]),
+        max_context=int(config.get("max_context", 1 << 20)),
+        checkpoint_dir=checkpoint_dir, loop=_loop(config, len(layers)),
+        loop_reenter=False, streams=streams,
         num_experts=max([(l.moe.experts if l.moe else 0) for l in layers]
                         + [0]))

@@ -83,8 +83,9 @@ class SectionedLinear(nn.Module):
 class LocalAttention(nn.Module):
     """Grouped-query softmax attention under a chunk and/or window mask, with
     per-head q/k RMS norm, rotation of a prefix of each head, split key and
-    value sizes, a per-head sigmoid output gate and an optional silent sink
-    in the softmax (each part can be switched off by the spec); the window may
+    value sizes, a sigmoid output gate (per head or elementwise) and an
+    optional sink in the softmax, silent or with a learned score per head
+    (each part can be switched off by the spec); the window may
     keep the first tokens, the rotation may use YaRN frequencies, and the
     values may be blended with those of the first blending layer of the step
     (which leaves them in `fb.aux`). Owns no
@@ -108,6 +109,12 @@ class LocalAttention(nn.Module):
         inv_freq, self.rot_amp = hops.yarn_inv_freq(
             spec.rot_dims, spec.rot_base, spec.rot_scaling)
         self.register_buffer("inv_freq", inv_freq, persistent=False)
+        if spec.sink_learned:
+            if not spec.sink:
+                raise ValueError("a learned sink is a sink")
+            self.sink_w = nn.Parameter(torch.zeros(spec.heads,
+                                                   dtype=torch.float32))
+        self.gate_n = spec.vdim if spec.gate_elements else 1
         if spec.v_mix:
             self.v_lambda = nn.Parameter(torch.zeros((), dtype=torch.float32))
 
@@ -117,12 +124,19 @@ class LocalAttention(nn.Module):
                 (tag + "k", s.kv_heads * s.dim, s.bias),
                 (tag + "v", s.kv_heads * s.vdim, s.bias)]
         if s.out_gate:
-            secs.append((tag + "g", s.heads, False))
+            secs.append((tag + "g", s.heads * self.gate_n, False))
         return secs
 
     @property
     def out_width(self) -> int:
         return self.spec.heads * self.spec.vdim
+
+    def param_targets(self, prefix: str, ck: str):
+        """Checkpoint tensors of this mixer that are not projections of the
+        sublayer input."""
+        if not self.spec.sink_learned:
+            return {}
+        return {ck + ".sink": (prefix + "sink_w", 0, 0, self.spec.heads, 1.0)}
 
     def kv_shape(self):
         return (self.spec.kv_heads, self.spec.dim, self.spec.vdim)
@@ -171,7 +185,8 @@ class LocalAttention(nn.Module):
             off[tag + "g"] if s.out_gate else -1, out, out_off, out_scale,
             token_seq=fb.token_seq, tile_seq=fb.tile_seq, tile_q0=fb.tile_q0,
             prefill_rows=fb.prefill_token_count, sink=s.sink,
-            keep_first=s.keep_first if s.window else 0)
+            keep_first=s.keep_first if s.window else 0, gate_n=self.gate_n,
+            sink_w=self.sink_w if s.sink_learned else None)
 
 
 class GatedDeltaRule(nn.Module):
@@ -463,7 +478,8 @@ class LatentAttention(nn.Module):
                 proj, off[tag + "dkv"], R, self.dkv_norm, self.eps,
                 _step_rope(fb, rd, s.rot_base, s.rot_scaling, self.inv_freq,
                            self.rot_amp),
-                cache.view(-1, R + rd), fb.slot_mapping, q, dk, qa)
+                cache.view(-1, R + rd), fb.slot_mapping, q, dk, qa,
+                adjacent=s.rot_adjacent)
         elif s.kv_from is None:
             hops.section_rmsnorm(proj, off[tag + "dkv"], R, self.dkv_norm,
                                  self.eps, cache.view(-1, R),
@@ -481,6 +497,26 @@ class LatentAttention(nn.Module):
                   out=sec.unflatten(1, (H, dv)).transpose(0, 1))
         if s.out_gate:
             hops.sigmoid_gate_mul(sec, proj, off[tag + "g"])
+
+
+class HyperConnection(nn.Module):
+    """The weights of one sublayer of a bundle of S residual streams: it reads
+    sum_s w_in[s] X_s, and its result y is written back as X_o <- sum_s
+    w_mix[s, o] X_s + w_out[o] y. (The op that writes a sublayer's result also
+    makes the next sublayer's input, so it needs two of these.)"""
+
+    def __init__(self, streams: int):
+        super().__init__()
+        f32 = torch.float32
+        self.w_in = nn.Parameter(torch.full((streams,), 1.0 / streams, dtype=f32))
+        self.w_out = nn.Parameter(torch.ones(streams, dtype=f32))
+        self.w_mix = nn.Parameter(torch.eye(streams, dtype=f32))
+
+    @staticmethod
+    def targets(prefix: str, ck: str, streams: int):
+        return {ck + ".in": (prefix + "w_in", 0, 0, streams, 1.0),
+                ck + ".out": (prefix + "w_out", 0, 0, streams, 1.0),
+                ck + ".mix": (prefix + "w_mix", 0, 0, streams, 1.0)}
 
 
 class MLSTM(nn.Module):
@@ -707,7 +743,8 @@ class SSDMixer(nn.Module):
 
 class RoutedExperts(nn.Module):
     """Mixture-of-experts feed-forward. The router runs in fp32: "sigmoid"
-    with group-limited choice and normalised weights, or "softmax" with a
+    with group-limited choice and weights that are the scores, normalised or
+    as they are, or "softmax" with a
     choice correction, identity experts and unnormalised scaled weights; or
     there is none ("table": a row of an integer table per token id, weights
     1 / top). Experts are `down act(up h)` ("relu2") or `down glu(gate h,
@@ -716,7 +753,9 @@ class RoutedExperts(nn.Module):
     run over the segments, and the caller folds the weighted sum of a token's
     rows into its residual kernel: forward returns (rows [padded rows, W],
     padpos [T, top], weights [T, top] or, when all are equal, one number,
-    identity weight [T] or None). A shared expert, if the spec has one, is
+    identity weight [T] or None). Where the weight multiplies an expert's
+    input, the first GEMM applies it to its products (they are linear in the
+    input) and the rows come back with weight 1. A shared expert, if the spec has one, is
     run by `shared_forward`. Where a table chooses, the layout depends on the
     token ids alone: it is made once a step and kept in `memo` (the step's
     scratch dict) for further runs of the same layer.
@@ -729,9 +768,14 @@ class RoutedExperts(nn.Module):
                  dtype: torch.dtype):
         super().__init__()
         if (spec.router, spec.act) not in (("sigmoid", "relu2"),
+                                           ("sigmoid", "silu_glu"),
                                            ("softmax", "clamped_glu"),
                                            ("table", "silu_glu")):
             raise ValueError("RoutedExperts: unknown router or activation")
+        if spec.weigh_input and (spec.router != "sigmoid"
+                                 or spec.act != "silu_glu"):
+            raise ValueError("weighted inputs go with the sigmoid router and "
+                             "silu units")
         self.spec = spec
         self.width = width
         E, ff = spec.experts, spec.ff
@@ -800,7 +844,7 @@ class RoutedExperts(nn.Module):
                 logits, self.correction if s.correction else None, s.top,
                 s.groups, s.keep, s.experts, s.route_scale)
         idx, wts = hops.moe_route(logits, s.top, s.groups, s.keep,
-                                  s.group_rank)
+                                  s.group_rank, s.renorm)
         return idx, wts, None
 
     def shared_forward(self, h: torch.Tensor):
@@ -821,6 +865,7 @@ class RoutedExperts(nn.Module):
         w1 = self.gate_up.view(s.experts, 2 * s.ff, self.width) if self.glu \
             else self.up
         bm = hops.expert_gemm_tile(h, w1, T * s.top)
+        row_w = None
         if s.router == "table":
             wts, idw = 1.0 / s.top, None
             layout = memo.get(("experts", id(self))) if memo is not None \
@@ -834,7 +879,10 @@ class RoutedExperts(nn.Module):
             # chosen identity experts share one segment past the real experts'
             # that no GEMM visits
             segs = s.experts + (1 if s.identity else 0)
-            layout = hops.moe_dispatch(idx, segs, bm)
+            layout = hops.moe_dispatch(idx, segs, bm,
+                                       wts if s.weigh_input else None)
+            if s.weigh_input:
+                layout, row_w, wts = layout[:4], layout[4], 1.0
         row_tok, tile_off, counts, padpos = layout
         tile_off, counts = tile_off[:s.experts + 1], counts[:s.experts]
         n = row_tok.shape[0]
@@ -842,7 +890,7 @@ class RoutedExperts(nn.Module):
         kind = {"relu2": hops.ACT_RELU2, "clamped_glu": hops.ACT_GLU_CLAMPED,
                 "silu_glu": hops.ACT_SILU_GATE}[s.act]
         hops.expert_gemm(act, h, w1, row_tok, tile_off, counts, kind, bm,
-                         s.limit)
+                         s.limit, row_w)
         rows = torch.empty((n, self.width), dtype=h.dtype, device=h.device)
         hops.expert_gemm(rows, act, self.down, None, tile_off, counts,
                          hops.ACT_NONE, bm)

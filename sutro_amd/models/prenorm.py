@@ -5,14 +5,21 @@
 with weighted RMS norms: the block and the model that the designs of this form
 share (which mixers, feed-forwards, embedding and head a model has is in its
 spec). A run of layers may be passed several times with the same weights
-(`spec.loop`): every pass has pages and state of its own, and the embedding
-output is added to the stream before each pass but the first.
+(`spec.loop`): every pass has pages and state of its own, and (by default) the
+embedding output is added to the stream before each pass but the first.
 
 The residual stream is fp32. Per sublayer: one merged input GEMM, the mixer's
 kernels, one output GEMM, and ONE kernel that adds the sublayer's result (for
 routed experts: the weighted gather of a token's expert rows, the identity
 share of its input and the shared expert; at the end of a pass: the embedding
 output) to the stream and emits the next sublayer's normed input.
+
+With `spec.streams` the residual is a bundle of streams (hyper-connections,
+`layers.HyperConnection`): a sublayer reads a weighted sum of them, and the
+same one kernel mixes the streams, adds the result to all of them and emits the
+next sublayer's normed input. The bundle is [T, streams, W] fp32; it is first
+written by the first layer's mixer (before that all streams are the embedding
+output) and the last sublayer of a step only makes the final normed sum.
 """
 
 from __future__ import annotations
@@ -32,14 +39,14 @@ from ..parallel.tp import TPContext
 from .hybrid_spec import (AttnMixerSpec, DecayAttnMixerSpec, DeltaMixerSpec,
                           HybridLayerSpec, HybridSpec, LatentAttnMixerSpec,
                           SSDMixerSpec)
-from .layers import (DecayAttention, GatedDeltaRule, LatentAttention,
-                     LocalAttention, RoutedExperts, SectionedLinear, SSDMixer,
-                     _pad)
+from .layers import (DecayAttention, GatedDeltaRule, HyperConnection,
+                     LatentAttention, LocalAttention, RoutedExperts,
+                     SectionedLinear, SSDMixer, _pad)
 
 
 class PreNormBlock(nn.Module):
     """One layer: norm, merged input projection, mixer, output projection;
-    norm, feed-forward (dense gated unit or routed experts)."""
+    norm, feed-forward (dense, gated or squared-ReLU, or routed experts)."""
 
     def __init__(self, spec: HybridSpec, layer: HybridLayerSpec, idx: int,
                  dtype: torch.dtype):
@@ -68,15 +75,29 @@ class PreNormBlock(nn.Module):
         self.out_padded = k != self.mixer.out_width
         self.out_proj = nn.Linear(k, W, bias=False, dtype=dtype)
         self.ff = layer.ff
+        self.relu2 = layer.ff_kind == "relu2"
         self.experts: Optional[RoutedExperts] = None
         if layer.ff or layer.moe is not None:
             self.norm2 = nn.Parameter(torch.ones(W, dtype=f32))
         if layer.ff:
             self.ff_in = SectionedLinear(
-                W, [("gate", layer.ff, False), ("up", layer.ff, False)], dtype)
+                W, [("up", layer.ff, False)] if self.relu2 else
+                [("gate", layer.ff, False), ("up", layer.ff, False)], dtype)
             self.ff_out = nn.Linear(layer.ff, W, bias=False, dtype=dtype)
         if layer.moe is not None:
             self.experts = RoutedExperts(layer.moe, W, dtype)
+        self.streams = spec.streams
+        self.hc1 = self.hc2 = None
+        if spec.streams:
+            self.hc1 = HyperConnection(spec.streams)
+            if self.has_ff:
+                self.hc2 = HyperConnection(spec.streams)
+            if layer.moe is not None and (
+                    layer.moe.identity
+                    or (layer.moe.shared_ff and layer.moe.shared_gate)):
+                raise ValueError(f"layer {idx}: several streams go with "
+                                 f"ungated shared experts, not with identity "
+                                 f"experts")
 
     @property
     def has_ff(self) -> bool:
@@ -98,28 +119,57 @@ class PreNormBlock(nn.Module):
                 if self.mixer.spec.v_mix else None
         t[ck + ".o"] = (prefix + "out_proj.weight", 1, 0,
                         self.mixer.out_width, 1.0)
-        if self.has_ff:
-            t[lp + ".norm2"] = (prefix + "norm2", 0, 0, W, 1.0, norm_offset)
+        # a layer without a feed-forward may still carry its (unused) norm and
+        # stream weights
+        t[lp + ".norm2"] = (prefix + "norm2", 0, 0, W, 1.0, norm_offset) \
+            if self.has_ff else None
+        for n, hc in (("hc1", self.hc1), ("hc2", self.hc2)):
+            if self.streams:
+                t.update(HyperConnection.targets(
+                    f"{prefix}{n}.", f"{lp}.{n}", self.streams)
+                    if hc is not None else
+                    {f"{lp}.{n}.{k}": None for k in ("in", "out", "mix")})
         if self.ff:
             t.update(self.ff_in.section_targets(
-                prefix + "ff_in.", {"gate": lp + ".mlp.gate",
-                                    "up": lp + ".mlp.up"}))
+                prefix + "ff_in.",
+                {n: f"{lp}.mlp.{n}" for n in self.ff_in.offsets}))
             t[lp + ".mlp.down"] = (prefix + "ff_out.weight", 1, 0, self.ff, 1.0)
         if self.experts is not None:
             t.update(self.experts.param_targets(prefix + "experts.",
                                                 lp + ".mlp"))
         return t
 
+    def _join(self, x: torch.Tensor, h: torch.Tensor,
+              hc: Optional[HyperConnection], norm_w: torch.Tensor,
+              next_in: Optional[torch.Tensor], x_in=None, extra=None,
+              write: bool = True, y=None, rows=None, padpos=None, wts=None,
+              idw=None, y2=None, proj2=None, sg: int = -1) -> None:
+        """Take a sublayer's result (y, expert rows, shared expert y2) into
+        the residual and make the next sublayer's input in h. One kernel."""
+        if hc is None:
+            # h is read (identity experts) and rewritten row by row
+            hops.add_rmsnorm(x, y, rows, padpos, wts, idw,
+                             h if idw is not None else None, y2, proj2, sg,
+                             norm_w, self.eps, h, x_in=x_in, extra=extra)
+        else:
+            hops.hyper_rmsnorm(x, x_in, y, rows, padpos, wts, y2, hc.w_mix,
+                               hc.w_out, next_in, norm_w, self.eps, h, write)
+
     def forward(self, x: torch.Tensor, h: torch.Tensor, fb: ForwardBatch,
                 kv: PagedKVCache, next_norm: torch.Tensor,
                 cache_idx: Optional[int] = None,
                 x_in: Optional[torch.Tensor] = None,
-                extra: Optional[torch.Tensor] = None) -> None:
+                extra: Optional[torch.Tensor] = None,
+                next_in: Optional[torch.Tensor] = None,
+                write: bool = True) -> None:
         """x fp32 [T, W]: the stream, updated in place (read from `x_in`
-        instead, if given). h [T, W] activation type: this layer's normed
+        instead, if given); with several streams [T, streams, W], each of
+        which is x_in, if given. h [T, W] activation type: this layer's normed
         input, overwritten with the next layer's (normed with the weight
-        `next_norm`). `cache_idx`: which pages or state this run uses.
-        `extra` fp32 [T, W]: joins the stream behind the layer."""
+        `next_norm`; with several streams their sum weighted by `next_in`).
+        `cache_idx`: which pages or state this run uses. `extra` fp32 [T, W]:
+        joins the stream behind the layer (single streams). `write` off:
+        nobody reads the streams behind this layer."""
         T = h.shape[0]
         proj = self.in_proj(h)
         alloc = torch.zeros if self.out_padded else torch.empty
@@ -131,18 +181,21 @@ class PreNormBlock(nn.Module):
         self.mixer(proj, self.in_proj.offsets, "", fb, kv, mix_in, 0, 1.0, **kw)
         y = self.out_proj(mix_in)
         if not self.has_ff:
-            hops.add_rmsnorm(x, y, norm_w=next_norm, eps=self.eps, h_out=h,
-                             x_in=x_in, extra=extra)
+            self._join(x, h, self.hc1, next_norm, next_in, x_in, extra, write,
+                       y=y)
             return
-        hops.add_rmsnorm(x, y, norm_w=self.norm2, eps=self.eps, h_out=h,
-                         x_in=x_in)
+        self._join(x, h, self.hc1, self.norm2,
+                   self.hc2.w_in if self.streams else None, x_in, y=y)
         if self.ff:
             proj = self.ff_in(h)
             off = self.ff_in.offsets
-            act = hops.glu_mul(proj, off["gate"], off["up"], self.ff,
-                               hops.GLU_SILU)
-            hops.add_rmsnorm(x, self.ff_out(act), norm_w=next_norm,
-                             eps=self.eps, h_out=h, extra=extra)
+            if self.relu2:
+                act = hops.relu_sq(proj)[:, :self.ff]
+            else:
+                act = hops.glu_mul(proj, off["gate"], off["up"], self.ff,
+                                   hops.GLU_SILU)
+            self._join(x, h, self.hc2, next_norm, next_in, None, extra, write,
+                       y=self.ff_out(act))
             return
         ex = self.experts
         rows, padpos, wts, idw = ex(h, fb.input_ids, fb.aux)
@@ -150,10 +203,9 @@ class PreNormBlock(nn.Module):
         sg = -1
         if ex.spec.shared_ff:
             y2, proj2, sg = ex.shared_forward(h)
-        # h is read (identity experts) and rewritten row by row in one kernel
-        hops.add_rmsnorm(x, None, rows, padpos, wts, idw,
-                         h if idw is not None else None, y2, proj2, sg,
-                         next_norm, self.eps, h, extra=extra)
+        self._join(x, h, self.hc2, next_norm, next_in, None, extra, write,
+                   rows=rows, padpos=padpos, wts=wts, idw=idw, y2=y2,
+                   proj2=proj2, sg=sg)
 
 
 class PreNormModel(nn.Module):
@@ -182,6 +234,9 @@ class PreNormModel(nn.Module):
             [PreNormBlock(spec, layer, i, dtype)
              for i, layer in enumerate(spec.layers)])
         self.final_norm = nn.Parameter(torch.ones(W, dtype=torch.float32))
+        if spec.streams:   # the model's output is the plain sum of the streams
+            self.register_buffer("sum_in", torch.ones(spec.streams),
+                                 persistent=False)
         if not spec.tie_embeddings:
             self.lm_head = nn.Linear(W, spec.vocab_size, bias=False, dtype=dtype)
         self.act_dtype = dtype
@@ -230,6 +285,8 @@ class PreNormModel(nn.Module):
                         device=e0.device)
         runs = s.runs
         n = len(runs)
+        if s.streams and n:
+            return self._forward_streams(e0, h, fb, kv)
         hops.add_rmsnorm(e0, norm_w=self.layers[runs[0][0]].norm1 if n
                          else self.final_norm, eps=s.norm_eps, h_out=h)
         # a looped model needs the embedding output again: the stream then
@@ -240,13 +297,36 @@ class PreNormModel(nn.Module):
             if j + 1 < n:
                 ni, npass = runs[j + 1]
                 nxt = self.layers[ni].norm1
-                if npass and ni == s.loop[0]:
+                if npass and ni == s.loop[0] and s.loop_reenter:
                     extra = e0
             self.layers[i](x, h, fb, kv, nxt, cache_idx=j,
                            x_in=e0 if j == 0 and s.loop else None, extra=extra)
             if self.layer_taps is not None:
                 self.layer_taps.append(x.clone() if extra is None
                                        else x - extra)
+        return h
+
+    def _forward_streams(self, e0: torch.Tensor, h: torch.Tensor,
+                         fb: ForwardBatch, kv: PagedKVCache) -> torch.Tensor:
+        """The layer runs over a bundle of streams (all of them e0 at first)."""
+        s = self.spec
+        runs = s.runs
+        x = torch.empty((e0.shape[0], s.streams, s.hidden_size),
+                        dtype=torch.float32, device=e0.device)
+        first = self.layers[runs[0][0]]
+        hops.hyper_rmsnorm(x, e0, in_w=first.hc1.w_in, norm_w=first.norm1,
+                           eps=s.norm_eps, h_out=h)
+        taps = self.layer_taps
+        for j, (i, _) in enumerate(runs):
+            last = j + 1 == len(runs)
+            nxt = None if last else self.layers[runs[j + 1][0]]
+            self.layers[i](
+                x, h, fb, kv, self.final_norm if last else nxt.norm1,
+                cache_idx=j, x_in=e0 if j == 0 else None,
+                next_in=self.sum_in if last else nxt.hc1.w_in,
+                write=not last or taps is not None)
+            if taps is not None:
+                taps.append(x.sum(dim=1))
         return h
 
     @torch.no_grad()
@@ -272,10 +352,21 @@ class PreNormModel(nn.Module):
                                    device=p.device) * std
 
             leaf = name.rsplit(".", 1)[-1]
-            if leaf in ("norm1", "norm2", "final_norm", "norm_w", "dkv_norm"):
+            if leaf in ("norm1", "norm2", "final_norm", "norm_w", "dkv_norm",
+                        "dq_norm"):
                 p.copy_(1.0 + rnd(p.shape, 0.05))
             elif leaf == "v_lambda":
                 p.fill_(0.3)
+            elif leaf == "sink_w":
+                p.copy_(rnd(p.shape, 0.5))
+            elif leaf == "w_in":    # streams: read about their mean,
+                p.copy_((1.0 + rnd(p.shape, 0.2)) / p.shape[0])
+            elif leaf == "w_out":   # written with about the full result,
+                p.copy_(1.0 + rnd(p.shape, 0.2))
+            elif leaf == "w_mix":   # mixed a little
+                S = p.shape[0]
+                p.copy_((torch.eye(S, device=p.device) + rnd(p.shape, 0.1))
+                        / (1.0 + 0.1 * S ** 0.5))
             elif leaf == "a_log":
                 p.copy_(rnd(p.shape, 0.3) - 0.5)
             elif leaf == "dt_bias":

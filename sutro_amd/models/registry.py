@@ -181,8 +181,8 @@ def spec_from_dir(path: str, name: Optional[str] = None):
     """Spec of a checkpoint directory, chosen by its ``config.json``.
 
     ``"architecture": "Vodinex"``, ``"Ruludra"``, ``"Vukotar"``,
-    ``"Nosalorn"`` or ``"Vanulorn"`` gives a layer-list :class:`HybridSpec`;
-    a Hugging-Face style ``"architectures": ["Qwen3...ForCausalLM"]`` gives a
+    ``"Nosalorn"``, ``"Vanulorn"`` or ``"Tubepel"`` gives a layer-list
+    :class:`HybridSpec`; a Hugging-Face style ``"architectures": ["Qwen3...ForCausalLM"]`` gives a
     :class:`ModelSpec` of the Qwen3 family. The returned spec remembers the
     directory, so engines built from it load its weights."""
     import json
@@ -219,6 +219,11 @@ def spec_from_dir(path: str, name: Optional[str] = None):
 
         return vanulorn_spec(cfg, name=name, checkpoint_dir=path,
                              tensor_shapes=safetensors_shapes(path))
+    if arch == "Tubepel":
+        from .hybrid_spec import tubepel_spec
+
+        return tubepel_spec(cfg, name=name, checkpoint_dir=path,
+                            tensor_shapes=safetensors_shapes(path))
     if arch and arch.startswith("Qwen3"):
         moe = int(cfg.get("num_experts", 0) or 0)
         heads = int(cfg["num_attention_heads"])
@@ -272,6 +277,10 @@ def build_model(spec, dtype, max_len: int, tp=None, moe_ep: bool = False):
         from .vanulorn import VanulornModel
 
         return VanulornModel(spec, dtype, max_len, tp)
+    if spec.arch == "tubepel":
+        from .tubepel import TubepelModel
+
+        return TubepelModel(spec, dtype, max_len, tp)
     from .qwen3 import Qwen3Model
 
     return Qwen3Model(spec, dtype, max_len, tp, moe_ep=moe_ep)

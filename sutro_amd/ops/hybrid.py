@@ -10,7 +10,8 @@ weighted RMS norms fused with the residual sum and the gather of expert rows,
 YaRN rotation tables, gated linear units, a softmax router with identity
 experts, and decay recurrences (fixed-decay linear attention, Mamba-2);
 rotated inputs of a decay recurrence, latents with a rotated key part, and
-experts chosen by a token table.
+experts chosen by a token table; hyper-connections (several residual streams)
+fused with the gather of expert rows and the next norm, and squared ReLU.
 
 GPU tensors run the HIP kernels of the `sutro_amd._C_mix` extension
 (csrc/mix_*.hip), templated on the activation type: bf16 when the engine
@@ -129,15 +130,19 @@ def local_attention(q, k_cache, v_cache, block_tables, seq_lens,
                     proj, gate_off: int, out, out_off: int, out_scale: float,
                     token_seq=None, tile_seq=None, tile_q0=None,
                     prefill_rows: int = 0, bias_r1=None, bias_r2=None,
-                    sink: bool = False, keep_first: int = 0):
+                    sink: bool = False, keep_first: int = 0,
+                    gate_n: int = 1, sink_w=None):
     """`tile_seq`/`tile_q0` (int32, 32 query rows a tile) cover the first
     `prefill_rows` rows: on the GPU in bf16 those rows run on the MFMA kernel
     when page size and head sizes allow it; the remaining (single-token) rows
     and all other cases run on the generic one-wave-per-row kernel.
     `bias_r1` / `bias_r2` (fp32 [H]): r1[h] * ln(1 + r2[h] * (i - j)) is taken
-    off the score of query i and key j. `sink`: a key of score 0 without a
-    value joins every row's normalisation (a one in the denominator).
-    `keep_first`: keys at positions below it stay visible past the window."""
+    off the score of query i and key j. `sink`: a score without key or value
+    joins every row's normalisation, 0 (a one in the denominator) or, with
+    `sink_w` (fp32 [H]), one learned number a head, not scaled.
+    `keep_first`: keys at positions below it stay visible past the window.
+    `gate_n`: gate columns a head at `gate_off`, 1 or the value size (one gate
+    an element)."""
     if q.is_cuda:
         if tile_seq is None or tile_seq.numel() == 0:
             tile_seq = tile_q0 = None
@@ -147,13 +152,14 @@ def local_attention(q, k_cache, v_cache, block_tables, seq_lens,
                                token_seq, scale, chunk, window, proj,
                                gate_off, out_scale, tile_seq, tile_q0,
                                prefill_rows, bias_r1, bias_r2, sink,
-                               keep_first)
+                               keep_first, gate_n, sink_w)
         return
     torch_ref.local_attention(q, k_cache, v_cache, block_tables, seq_lens,
                               query_start_locs, scale, chunk, window, proj,
                               gate_off, out, out_off, out_scale,
                               bias_r1=bias_r1, bias_r2=bias_r2, sink=sink,
-                              keep_first=keep_first)
+                              keep_first=keep_first, gate_n=gate_n,
+                              sink_w=sink_w)
 
 
 def delta_prep(proj, q_off, k_off, v_off, b_off, a1_off, H, G, dk, dv,
@@ -339,23 +345,26 @@ def dyt_residual(x, y1=None, ls1=None, y2=None, ls2=None, rows=None,
                            nb, h_out if norm is not None else None)
 
 
-def moe_route(logits, top: int, groups: int, keep: int, group_rank: int = 2):
+def moe_route(logits, top: int, groups: int, keep: int, group_rank: int = 2,
+              renorm: bool = True):
     """Sigmoid router with group-limited choice over fp32 logits [T, E]:
-    (idx int32 [T, top], weights fp32 [T, top])."""
+    (idx int32 [T, top], weights fp32 [T, top]); the weights are the chosen
+    scores, divided by their sum if `renorm`."""
     if logits.is_cuda:
         T = logits.shape[0]
         idx = torch.empty((T, top), dtype=torch.int32, device=logits.device)
         w = torch.empty((T, top), dtype=torch.float32, device=logits.device)
-        _mix().moe_route(idx, w, logits, groups, keep, group_rank)
+        _mix().moe_route(idx, w, logits, groups, keep, group_rank, renorm)
         return idx, w
-    return torch_ref.moe_route(logits, top, groups, keep, group_rank)
+    return torch_ref.moe_route(logits, top, groups, keep, group_rank, renorm)
 
 
-def moe_dispatch(idx, experts: int, bm: int):
+def moe_dispatch(idx, experts: int, bm: int, wts=None):
     """Per-expert segments padded to `bm` rows for idx int32 [T, k]:
     (row_tok int32 [(ceil(T*k / bm) + experts) * bm], tile_off int32
-    [experts+1], counts int32 [experts], padpos int32 [T, k]). One kernel, no
-    host round trip."""
+    [experts+1], counts int32 [experts], padpos int32 [T, k]). No host round
+    trip. With `wts` (fp32 [T, k]) a fifth item: the weight of every row (fp32,
+    0 for padding)."""
     if idx.is_cuda:
         T, k = idx.shape
         dev = idx.device
@@ -364,9 +373,18 @@ def moe_dispatch(idx, experts: int, bm: int):
         tile_off = torch.empty(experts + 1, dtype=torch.int32, device=dev)
         counts = torch.empty(experts, dtype=torch.int32, device=dev)
         padpos = torch.empty((T, k), dtype=torch.int32, device=dev)
-        _mix().moe_dispatch(row_tok, tile_off, counts, padpos, idx, bm)
-        return row_tok, tile_off, counts, padpos
-    return torch_ref.moe_dispatch(idx, experts, bm)
+        row_w = None if wts is None else torch.empty(
+            row_tok.shape, dtype=torch.float32, device=dev)
+        _mix().moe_dispatch(row_tok, tile_off, counts, padpos, idx, bm, wts,
+                            row_w)
+        layout = (row_tok, tile_off, counts, padpos)
+        return layout if wts is None else layout + (row_w,)
+    layout = torch_ref.moe_dispatch(idx, experts, bm)
+    if wts is None:
+        return layout
+    row_w = torch.zeros(layout[0].shape, dtype=torch.float32, device=idx.device)
+    row_w[layout[3].long().reshape(-1)] = wts.reshape(-1)
+    return layout + (row_w,)
 
 
 def expert_gemm_tile(a, w, n_rows: int) -> int:
@@ -381,21 +399,23 @@ def expert_gemm_tile(a, w, n_rows: int) -> int:
 
 
 def expert_gemm(out, a, w, row_tok, tile_off, counts, act: int, bm: int,
-                limit: float = 0.0):
+                limit: float = 0.0, row_w=None):
     """out[r] = act(a[row_tok[r]] @ w[e(r)]^T) over padded per-expert
     segments (row_tok None: a is already laid out in segments). w [E, N, K];
     act: ACT_NONE, ACT_RELU2, or a gated unit (w holds N/2 gate rows then
     N/2 up rows per expert, out is N/2 wide): ACT_SILU_GATE silu(gate) up;
     ACT_GLU_CLAMPED g sigmoid(1.702 g) (u + 1) with g = min(gate, limit), u =
-    clamp(up, -limit, limit)."""
+    clamp(up, -limit, limit). `row_w` (fp32, one a row; gated units): the
+    expert reads row_w[r] * a[row_tok[r]] (applied to the products)."""
     if out.is_cuda:
         _mix().expert_gemm(out, a, w, row_tok, tile_off, counts, act, bm,
-                           limit)
+                           limit, row_w)
         return out
     if act in (ACT_GLU_CLAMPED, ACT_SILU_GATE):
         return torch_ref.glu_grouped_gemm(out, a, w, row_tok, tile_off,
                                           counts, bm, limit,
-                                          silu=act == ACT_SILU_GATE)
+                                          silu=act == ACT_SILU_GATE,
+                                          row_w=row_w)
     return torch_ref.grouped_gemm(out, a, w, row_tok, tile_off, counts,
                                   out.shape[0] // bm, act, bm)
 
@@ -561,16 +581,17 @@ def rotary_sections(proj, offs, H: int, dk: int, dv: int, cos_sin,
 
 
 def latent_prep(proj, off: int, R: int, norm_w, eps: float, cos_sin, cache,
-                rows, q, q_off: int, qa) -> None:
+                rows, q, q_off: int, qa, adjacent: bool = False) -> None:
     """One kernel per latent layer with a rotated key part: the normed latent
     and the rotated key part into cache row rows[t] ([N, R + rd]), the rotated
-    query parts q[t, h, q_off : q_off + rd] into qa[t, h, R:]."""
+    query parts q[t, h, q_off : q_off + rd] into qa[t, h, R:]. Pairs (i, i +
+    rd/2) turn together, or neighbours (2i, 2i + 1) if `adjacent`."""
     if proj.is_cuda:
         _mix().latent_prep(proj, off, norm_w, eps, cos_sin, cache, rows, q,
-                           q_off, qa)
+                           q_off, qa, adjacent)
         return
     torch_ref.latent_prep(proj, off, R, norm_w, eps, cos_sin, cache, rows, q,
-                          q_off, qa)
+                          q_off, qa, adjacent)
 
 
 def moe_dispatch_table(ids, table, experts: int, bm: int):
@@ -588,3 +609,33 @@ def moe_dispatch_table(ids, table, experts: int, bm: int):
                                   table, bm)
         return row_tok, tile_off, counts, padpos
     return torch_ref.moe_dispatch(table[ids], experts, bm)
+
+
+# ---- hyper-connections, squared ReLU ----
+
+
+def hyper_rmsnorm(x, x_in=None, y=None, rows=None, padpos=None, wts=None,
+                  y2=None, mix=None, out=None, in_w=None, norm_w=None,
+                  eps: float = 1e-6, h_out=None, write: bool = True) -> None:
+    """Streams x (fp32 [T, S, W]; all equal to x_in [T, W], if given): with
+    `mix` [from, to] and `out`, X_o <- sum_s mix[s, o] X_s + out[o] r where r =
+    y + sum_j wts[t, j] rows[padpos[t, j]] + y2 (each optional; `wts` may be
+    one number for all pairs), written back unless `write` is off; then h_out =
+    u / sqrt(mean(u^2) + eps) * norm_w with u = sum_s in_w[s] X_s. One
+    kernel."""
+    if x.is_cuda:
+        same = rows is not None and not torch.is_tensor(wts)
+        _mix().hyper_rmsnorm(x, x_in, y, rows, padpos, None if same else wts,
+                             float(wts) if same else 0.0, y2, mix, out, in_w,
+                             norm_w, eps, h_out, write)
+        return
+    torch_ref.hyper_rmsnorm(x, x_in, y, rows, padpos, wts, y2, mix, out, in_w,
+                            norm_w, eps, h_out, write)
+
+
+def relu_sq(z):
+    """max(z, 0)^2, in place."""
+    if z.is_cuda:
+        _mix().relu_sq(z)
+        return z
+    return torch_ref.relu_sq(z)

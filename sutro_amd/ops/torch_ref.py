@@ -269,7 +269,8 @@ def attn_prep(proj, q_off, k_off, v_off, H, G, dk, dv, q_norm_w, k_norm_w,
 def local_attention(q, k_cache, v_cache, block_tables, seq_lens,
                     query_start_locs, scale, chunk, window, proj, gate_off,
                     out, out_off, out_scale, bias_r1=None, bias_r2=None,
-                    sink=False, keep_first: int = 0):
+                    sink=False, keep_first: int = 0, gate_n: int = 1,
+                    sink_w=None):
     """Softmax attention of each sequence's new tokens over its cached keys
     under a local mask: query at position i sees j <= i with
     j >= (i // chunk) * chunk (chunk > 0) and j > i - window (window > 0);
@@ -277,8 +278,10 @@ def local_attention(q, k_cache, v_cache, block_tables, seq_lens,
     Head h's result is multiplied by out_scale * sigmoid(proj[t, gate_off+h])
     (gate_off < 0: no gate) and written to out[t, out_off + h*dv : ...].
     With bias_r1 / bias_r2 (fp32 [H]) the score of query i and key j is
-    lowered by r1[h] * ln(1 + r2[h] * (i - j)). With `sink` a key of score 0
-    that carries no value joins the normalisation."""
+    lowered by r1[h] * ln(1 + r2[h] * (i - j)). With `sink` a score without
+    key or value (0, or sink_w[h]) joins the normalisation. `gate_n` = dv: the
+    gate has an element of its own for every element of the result, head h's
+    start at gate_off + h*dv."""
     T, H, dk = q.shape
     G, bs, dv = v_cache.shape[1], v_cache.shape[2], v_cache.shape[3]
     rep = H // G
@@ -310,14 +313,17 @@ def local_attention(q, k_cache, v_cache, block_tables, seq_lens,
             hidden = hidden | ((kpos <= qpos - window) & (kpos >= keep_first))
         scores.masked_fill_(hidden.unsqueeze(0), float("-inf"))
         if sink:
-            zero = torch.zeros(H, nq, 1, dtype=scores.dtype, device=q.device)
-            pr = torch.softmax(torch.cat([scores, zero], -1), dim=-1)[..., :L]
+            extra = torch.zeros(H, nq, 1, dtype=scores.dtype, device=q.device)
+            if sink_w is not None:
+                extra += sink_w.float().view(H, 1, 1)
+            pr = torch.softmax(torch.cat([scores, extra], -1), dim=-1)[..., :L]
         else:
             pr = torch.softmax(scores, dim=-1)
         o = torch.einsum("hqk,hkd->hqd", pr, vh)
         o = o.transpose(0, 1) * out_scale                      # [nq, H, dv]
         if gate_off >= 0:
-            o = o * torch.sigmoid(proj[q0:q1, gate_off:gate_off + H].float()).unsqueeze(-1)
+            g = proj[q0:q1, gate_off:gate_off + H * gate_n].float()
+            o = o * torch.sigmoid(g).view(nq, H, gate_n)
         out[q0:q1, out_off:out_off + H * dv] = o.reshape(nq, H * dv).to(out.dtype)
 
 
@@ -626,12 +632,13 @@ def dyt_residual(x, y1, ls1, y2, ls2, rows, padpos, wts, alpha, nw, nb,
         h_out.copy_((torch.tanh(alpha * x) * nw + nb).to(h_out.dtype))
 
 
-def moe_route(logits, top: int, groups: int, keep: int, group_rank: int = 2):
+def moe_route(logits, top: int, groups: int, keep: int, group_rank: int = 2,
+              renorm: bool = True):
     """Sigmoid router with group-limited choice. logits fp32 [T, E]. Returns
     (idx int32 [T, top], weights fp32 [T, top]): the `top` largest sigmoid
     scores among the experts of the `keep` groups (equal runs of neighbours)
-    whose `group_rank` largest scores sum highest, each divided by the sum of
-    the chosen scores + 1e-20. Ties go to the lower index."""
+    whose `group_rank` largest scores sum highest, with `renorm` each divided
+    by the sum of the chosen scores + 1e-20. Ties go to the lower index."""
     T, E = logits.shape
     s = torch.sigmoid(logits.float())
     if groups > 1:
@@ -649,7 +656,8 @@ def moe_route(logits, top: int, groups: int, keep: int, group_rank: int = 2):
     idx = torch.sort(masked, dim=-1, descending=True,
                      stable=True).indices[:, :top]
     w = s.gather(1, idx)
-    w = w / (w.sum(-1, keepdim=True) + 1e-20)
+    if renorm:
+        w = w / (w.sum(-1, keepdim=True) + 1e-20)
     return idx.to(torch.int32), w
 
 
@@ -814,11 +822,11 @@ def moe_route_softmax(logits, corr, top: int, groups: int, keep: int,
 
 
 def glu_grouped_gemm(out, a, w, row_tok, tile_off, counts, bm: int,
-                     limit: float, silu: bool = False):
+                     limit: float, silu: bool = False, row_w=None):
     """Per-expert segments like `grouped_gemm`, gathered rows, w [E, 2*ff, K]
     holding gate rows then up rows; out[r] = g sigmoid(1.702 g) (u + 1) with
     g = min(gate, limit), u = clamp(up, -limit, limit); or, with `silu`,
-    silu(gate) up."""
+    silu(gate) up. Row r reads row_w[r] times its input, if given."""
     E, N, K = w.shape
     ff = N // 2
     for e in range(E):
@@ -827,6 +835,8 @@ def glu_grouped_gemm(out, a, w, row_tok, tile_off, counts, bm: int,
             continue
         s0 = int(tile_off[e]) * bm
         rows = a[row_tok[s0:s0 + c].long().clamp(min=0)].float()
+        if row_w is not None:
+            rows = rows * row_w[s0:s0 + c].unsqueeze(1)
         if silu:
             g = rows @ w[e, :ff].T.float()
             u = rows @ w[e, ff:].T.float()
@@ -961,12 +971,17 @@ def gated_group_norm(o, proj, g_off: int, norm_w, eps: float, groups: int,
 # --------------------------------------------------------------------------
 
 
-def _rotate_prefix(x, cos_sin):
+def _rotate_prefix(x, cos_sin, adjacent: bool = False):
     """x fp32 [T, heads, d]: the first 2 * half dimensions of every head are
-    rotated in pairs (i, i + half); cos_sin fp32 [T, 2 * half] = cos | sin."""
+    rotated in pairs (i, i + half), or (2i, 2i + 1) if `adjacent`; cos_sin
+    fp32 [T, 2 * half] = cos | sin."""
     half = cos_sin.shape[1] // 2
     c = cos_sin[:, :half].unsqueeze(1)
     s = cos_sin[:, half:].unsqueeze(1)
+    if adjacent:
+        u, v = x[..., 0:2 * half:2], x[..., 1:2 * half:2]
+        y = torch.stack([u * c - v * s, v * c + u * s], dim=-1).flatten(-2)
+        return torch.cat([y, x[..., 2 * half:]], dim=-1)
     u, v = x[..., :half], x[..., half:2 * half]
     return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * half:]], dim=-1)
 
@@ -987,14 +1002,53 @@ def rotary_sections(proj, offs, H: int, dk: int, dv: int, cos_sin,
 
 
 def latent_prep(proj, off: int, R: int, norm_w, eps: float, cos_sin, cache,
-                rows, q, q_off: int, qa) -> None:
+                rows, q, q_off: int, qa, adjacent: bool = False) -> None:
     """cache [N, R + rd] row rows[t] = (n(proj[t, off : off+R]) * norm_w) |
     rotated(proj[t, off+R : off+R+rd]); qa[t, h, R:] = rotated(q[t, h,
-    q_off : q_off+rd]), rd = the width of cos_sin."""
+    q_off : q_off+rd]), rd = the width of cos_sin. `adjacent`: neighbours
+    (2i, 2i + 1) turn together instead of (i, i + rd/2)."""
     rd = cos_sin.shape[1]
     c = _unit_rms(proj[:, off:off + R].float(), eps) * norm_w.float()
     kr = _rotate_prefix(proj[:, off + R:off + R + rd].float().unsqueeze(1),
-                        cos_sin).squeeze(1)
+                        cos_sin, adjacent).squeeze(1)
     cache[rows] = torch.cat([c, kr], dim=1).to(cache.dtype)
     qa[..., R:] = _rotate_prefix(q[..., q_off:q_off + rd].float(),
-                                 cos_sin).to(qa.dtype)
+                                 cos_sin, adjacent).to(qa.dtype)
+
+
+# ---- hyper-connections, squared ReLU ----
+
+
+def hyper_rmsnorm(x, x_in, y, rows, padpos, wts, y2, mix, out, in_w, norm_w,
+                  eps: float, h_out, write: bool = True) -> None:
+    """x fp32 [T, S, W] streams (all equal to x_in [T, W], if given). With
+    `mix` [from, to] and `out` [S]: X_o <- sum_s mix[s, o] X_s + out[o] r, r =
+    y + sum_j wts[t, j] rows[padpos[t, j]] + y2 (each optional; wts may be one
+    number), in place unless `write` is off. Then h_out = u / sqrt(mean(u^2) +
+    eps) * norm_w, u = sum_s in_w[s] X_s, unless h_out is None."""
+    T, S, W = x.shape
+    X = x if x_in is None else x_in.unsqueeze(1).expand(T, S, W)
+    if mix is not None:
+        r = torch.zeros(T, W, dtype=torch.float32, device=x.device)
+        if y is not None:
+            r = r + y.float()
+        if rows is not None:
+            picked = rows[padpos.long()].float()
+            r = r + ((picked * wts.unsqueeze(-1)).sum(1)
+                     if torch.is_tensor(wts) else picked.sum(1) * wts)
+        if y2 is not None:
+            r = r + y2.float()
+        X = torch.einsum("tsw,so->tow", X, mix) \
+            + out.view(1, S, 1) * r.unsqueeze(1)
+        if write:
+            x.copy_(X)
+    if h_out is not None:
+        u = torch.einsum("tsw,s->tw", X, in_w)
+        h_out.copy_((u * torch.rsqrt(u.pow(2).mean(-1, keepdim=True) + eps)
+                     * norm_w.float()).to(h_out.dtype))
+
+
+def relu_sq(z):
+    """max(z, 0)^2 (fp32 math), in place."""
+    r = torch.relu(z.float())
+    return z.copy_((r * r).to(z.dtype))
