@@ -242,7 +242,13 @@ def make_config(width, vocab, layers, streams=2, loop=None, eps=1e-5):
 
 
 def make_weights(config, seed=0):
-    """Random weights (already rounded to bf16) under checkpoint names."""
+    """Random weights (already rounded to bf16) under checkpoint names.
+
+    Which experts a token uses must not hang on rounding, or bf16 runs could
+    not be compared: the first columns (one per expert) are written by no
+    sublayer, every token's embedding holds well separated numbers there in an
+    order of its own, and router row e looks at column e alone. The scores
+    still depend on everything that scales the normed input."""
     g = torch.Generator().manual_seed(seed)
     W, S = config["width"], config["streams"]
     w = {}
@@ -254,10 +260,16 @@ def make_weights(config, seed=0):
         return rnd(out, inn, std=gain * inn ** -0.5)
 
     def swi(p, ff):
-        w[p + "gate"], w[p + "up"] = lin(ff, W, 1.5), lin(ff, W, 1.5)
+        w[p + "gate"], w[p + "up"] = lin(ff, W), lin(ff, W)
         w[p + "down"] = lin(W, ff)
 
     w["embed"], w["head"] = rnd(config["vocab"], W), lin(config["vocab"], W)
+    E = max([(lc.get("mlp") or {}).get("router", {}).get("experts", 0)
+             for lc in config["layers"]])
+    if E:
+        levels = torch.linspace(-1.5, 1.5, E)
+        for t in range(config["vocab"]):
+            w["embed"][t, :E] = levels[torch.randperm(E, generator=g)]
     w["final.norm"] = rnd(W, std=0.2, mean=1.0)
     for i, lc in enumerate(config["layers"]):
         lp, mc, fc = f"l{i}.", lc["mixer"], lc.get("mlp")
@@ -272,16 +284,16 @@ def make_weights(config, seed=0):
         H, dk, dv = mc["heads"], mc["dim"], mc["vdim"]
         if lc["type"] == "attention":
             G = mc["kv_heads"]
-            w[p + "q"], w[p + "k"] = lin(H * dk, W, 1.5), lin(G * dk, W, 1.5)
+            w[p + "q"], w[p + "k"] = lin(H * dk, W), lin(G * dk, W)
             w[p + "v"], w[p + "g"] = lin(G * dv, W), lin(H * dv, W, 2.0)
             w[p + "sink"] = rnd(H, std=1.0, mean=1.0)
         else:
             R, Q, dr = mc["kv_rank"], mc["q_rank"], mc["rot_dim"]
             w[p + "dq"], w[p + "dq.norm"] = lin(Q, W), rnd(Q, std=0.2, mean=1.0)
-            w[p + "uq"] = lin(H * (dk + dr), Q, 1.5)
-            w[p + "dkv"] = lin(R + dr, W, 1.5)
+            w[p + "uq"] = lin(H * (dk + dr), Q)
+            w[p + "dkv"] = lin(R + dr, W)
             w[p + "dkv.norm"] = rnd(R, std=0.2, mean=1.0)
-            w[p + "uk"], w[p + "uv"] = lin(H * dk, R, 1.5), lin(H * dv, R)
+            w[p + "uk"], w[p + "uv"] = lin(H * dk, R), lin(H * dv, R)
         w[p + "o"] = lin(W, H * dv)
         if fc is None:
             continue
@@ -289,11 +301,17 @@ def make_weights(config, seed=0):
         if fc["kind"] == "dense":
             w[m + "up"], w[m + "down"] = lin(fc["ff"], W), lin(W, fc["ff"])
             continue
-        w[m + "router"] = lin(fc["router"]["experts"], W, 1.5)
+        n = fc["router"]["experts"]
+        w[lp + "norm2"][:E] = 1.0
+        w[m + "router"] = torch.zeros(n, W)
+        w[m + "router"][:, :n] = 1.5 * torch.eye(n)
         for e in range(fc["router"]["experts"]):
             swi(f"{m}e{e}.", fc["expert"]["ff"])
         if fc.get("shared"):
             swi(m + "shared.", fc["shared"]["ff"])
+    for k, v in w.items():
+        if k.endswith((".o", ".down")):
+            v[:E] = 0.0
     return {k: v.to(torch.bfloat16).to(F64) for k, v in w.items()}
 
 
