@@ -79,9 +79,9 @@ def build_args():
                         "of 1b,8b,tiny); one JSON line per model")
     p.add_argument("--compare-models", type=str, default="vodinex,qwen3",
                    help="models of --arch-compare: comma list of vodinex, "
-                        "ruludra, vukotar, nosalorn, vanulorn, qwen3, qwen3moe "
-                        "(the counterpart of those with routed experts is "
-                        "qwen3moe)")
+                        "ruludra, vukotar, nosalorn, vanulorn, tubepel, qwen3, "
+                        "qwen3moe (the counterpart of those with routed "
+                        "experts)")
     p.add_argument("--compare-seqs", type=int, default=16)
     p.add_argument("--compare-prompt", type=int, default=2048)
     p.add_argument("--e2e-rows", type=int, default=3000,

@@ -1,6 +1,7 @@
 """Prefill and decode throughput of the layer-list decoders (Vodinex,
-Ruludra, Vukotar, Nosalorn, Vanulorn) beside the Qwen3 decoder of equal size (same width, layers,
-heads, key/value heads, head size and feed-forward width; for Vukotar the
+Ruludra, Vukotar, Nosalorn, Vanulorn, Tubepel) beside the Qwen3 decoder of
+equal size (same width, layers, heads, key/value heads, head size and
+feed-forward width; for Vukotar the
 Qwen3 mixture-of-experts decoder with as many experts of the same inner
 width and as many choices a token), all with random weights, all through the
 engine's own batch path (scheduler, paged cache, state slots, decode
@@ -196,6 +197,43 @@ def looped_spec(name: str) -> HybridSpec:
                       tie_embeddings=True, num_experts=MOE_EXPERTS)
 
 
+def streams_spec(name: str, window: int = 1024) -> HybridSpec:
+    """Tubepel at the same width, depth (layer runs), heads and head size, with
+    four residual streams: a rotary latent attention (query latent W/2, latent
+    4 head sizes, rotated part half a head) with a squared-ReLU feed-forward,
+    a windowed attention (as many key/value heads, kept first tokens, sinks,
+    elementwise gate) and a second latent attention (the other pairing) that
+    are passed twice and once, both beside 32 SwiGLU experts (4 a token, inner
+    width ff/4, weighted inputs) and a shared expert of the same width."""
+    W, L, H, G, D, ff, V = SIZES[name]
+
+    def lat(adjacent: bool) -> LatentAttnMixerSpec:
+        return LatentAttnMixerSpec(
+            heads=H, dim=D, vdim=D, q_rank=W // 2, kv_rank=4 * D,
+            scale=(D + D // 2) ** -0.5, rot_dim=D // 2, rot_base=10000.0,
+            out_gate=False, rot_adjacent=adjacent)
+
+    attn = AttnMixerSpec(heads=H, kv_heads=G, dim=D, vdim=D, scale=D ** -0.5,
+                         rot_dims=D // 2, rot_base=500000.0, window=window,
+                         keep_first=4, qk_norm=False, bias=False,
+                         gate_elements=True, sink=True, sink_learned=True)
+    eff = max(64, ff // MOE_FF_DIV)
+    moe = RoutedExpertsSpec(ff=eff, experts=MOE_EXPERTS, top=MOE_TOP,
+                            router="sigmoid", act="silu_glu", shared_ff=eff,
+                            shared_gate=False, renorm=False, weigh_input=True)
+    layers = [HybridLayerSpec("latent_attention_2", lat(False), ff=ff,
+                              ff_kind="relu2"),
+              HybridLayerSpec("attention", attn, ff_kind="relu2", moe=moe),
+              HybridLayerSpec("latent_attention", lat(True), ff_kind="relu2",
+                              moe=moe)]
+    layers = layers[:L]
+    loop = (1, 2, L - 2) if L > 3 else None
+    return HybridSpec(name=f"tubepel-{name}", arch="tubepel", hidden_size=W,
+                      vocab_size=V, layers=tuple(layers), norm_eps=1e-6,
+                      max_context=1 << 20, loop=loop, loop_reenter=False,
+                      streams=4, num_experts=MOE_EXPERTS)
+
+
 def moe_spec(name: str) -> ModelSpec:
     """The Qwen3 mixture-of-experts decoder with as many experts of the same
     inner width and as many choices a token (softmax router, SwiGLU
@@ -269,7 +307,7 @@ def _measure(spec, device: str, seqs: int, prompt: int, steps: int,
 MAKERS = {"vodinex": hybrid_spec, "qwen3": dense_spec,
           "ruludra": sandwich_spec, "vukotar": parallel_spec,
           "qwen3moe": moe_spec, "nosalorn": prenorm_spec,
-          "vanulorn": looped_spec}
+          "vanulorn": looped_spec, "tubepel": streams_spec}
 
 
 def run_compare(sizes: List[str], device: str, seqs: int, prompt: int,
